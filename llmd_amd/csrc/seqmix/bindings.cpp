@@ -40,25 +40,30 @@ int sm_selective_scan(const void*, const void*, const void*, const float*, const
 int sm_gdelta_scan(const void*, int64_t, const void*, const void*, const void*, const void*, float, int, int, float*,
                    const int*, const int*, const int*, void*, int, int, hipStream_t);
 void sm_hyper_embed(const int64_t*, const void*, int64_t, float*, int, int, int, int, hipStream_t);
-void sm_hyper_norm(const float*, const float*, const void*, float, void*, int, int, int, int, hipStream_t);
+void sm_hyper_norm(const float*, const float*, const void*, float, void*, int, int, int, int, int, hipStream_t);
 void sm_hyper_update_norm(float*, const void*, int64_t, const float*, const float*, const float*, const void*, float,
-                          void*, int, int, int, int, hipStream_t);
-void sm_gated_act(const void*, int64_t, int, int, void*, int, int, hipStream_t);
+                          void*, int, int, int, int, int, hipStream_t);
+void sm_gated_act(const void*, int64_t, int, int, void*, int, int, float, hipStream_t);
 void sm_qkv_rope_cache(const void*, int64_t, const float*, const int64_t*, const float*, int, int, int, int, int, int,
                        int, float, float*, int, float, const int64_t*, void*, int, void*, const float*, int, int, int,
-                       int, const void*, void*, int, const int*, const int*, const int*, const int*, int, int,
-                       hipStream_t);
+                       int, const void*, void*, int, const int*, const int*, const int*, const int*, int, int, int,
+                       const float*, hipStream_t);
 int sm_grouped_attention(const void*, const void*, const int*, int, int, const int*, const int*, float, int, int, int,
                          int, int, int, const void*, int64_t, void*, int, const float*, int, const float*, int, int,
                          hipStream_t);
 int sm_grouped_attention_mfma(const void*, const void*, const int*, int, int, const int*, int, const int*, float, int,
                               int, int, int, const void*, int64_t, void*, int, int, float*, float*, int, const float*,
                               int, const float*, int, int, int, hipStream_t);
-void sm_moe_route_scores(const float*, const float*, int, int, int*, float*, int, hipStream_t);
+void sm_moe_route_scores(const float*, const float*, int, int, int*, float*, int, int, int, float, hipStream_t);
 void sm_moe_route(const float*, int64_t, int, int, int*, float*, int, int, hipStream_t);
 void sm_moe_group(const int*, int, int, int*, int*, int*, int, hipStream_t);
 void sm_moe_gemm(const void*, int64_t, int, const int*, const int*, const void*, int, int, void*, int, int, int, int,
-                 const float*, hipStream_t);
+                 const float*, float, hipStream_t);
+int sm_retention(const void*, int64_t, int, int, int, int, const int64_t*, const float*, int, const float*, int, float,
+                 float*, const int*, const int*, const int*, void*, int, int, int, int, int, const int*, const int*,
+                 float*, float*, hipStream_t);
+int sm_retention_chunk();
+int sm_retention_cols();
 void sm_bigram_embed(const int64_t*, const void*, float, int64_t, const void*, int64_t, int64_t, int64_t, int*,
                      const int*, const int*, const int*, const int*, int*, float*, void*, int, int, int, hipStream_t);
 void sm_post_norm_add(const void*, int64_t, const void*, int64_t, float, float, const float*, const void*, float*, float,
@@ -359,7 +364,7 @@ void check_streams(const Tensor& X) {
   TORCH_CHECK(X.dim() == 3 && X.size(0) >= 1 && X.size(0) <= 16 && X.size(2) <= 16384, "X [S <= 16, T, d <= 16384]");
 }
 
-void hyper_norm(Tensor X, Tensor w_in, Tensor norm_w, double eps, Tensor out) {
+void hyper_norm(Tensor X, Tensor w_in, Tensor norm_w, double eps, Tensor out, bool rms) {
   const c10::hip::OptionalHIPGuard g(dev_of(X));
   check_streams(X);
   CHECK_F32(w_in);
@@ -369,11 +374,11 @@ void hyper_norm(Tensor X, Tensor w_in, Tensor norm_w, double eps, Tensor out) {
   CHECK_ACT(out, norm_w);
   TORCH_CHECK(out.is_contiguous() && out.dim() == 2 && out.size(0) == T && out.size(1) == d, "out [T, d]");
   sm_hyper_norm(X.data_ptr<float>(), w_in.data_ptr<float>(), norm_w.data_ptr(), (float)eps, out.data_ptr(), S, T, d,
-                is_f32(norm_w), cur());
+                rms ? 1 : 0, is_f32(norm_w), cur());
 }
 
 void hyper_update_norm(Tensor X, Tensor y, Tensor mix, Tensor w_out, std::optional<Tensor> next_in,
-                       std::optional<Tensor> next_w, double eps, std::optional<Tensor> out) {
+                       std::optional<Tensor> next_w, double eps, std::optional<Tensor> out, bool rms) {
   const c10::hip::OptionalHIPGuard g(dev_of(X));
   check_streams(X);
   CHECK_F32(mix);
@@ -396,30 +401,32 @@ void hyper_update_norm(Tensor X, Tensor y, Tensor mix, Tensor w_out, std::option
     o = out->data_ptr();
   }
   sm_hyper_update_norm(X.data_ptr<float>(), y.data_ptr(), y.stride(0), mix.data_ptr<float>(), w_out.data_ptr<float>(),
-                       nin, nw, (float)eps, o, S, T, d, is_f32(y), cur());
+                       nin, nw, (float)eps, o, S, T, d, rms ? 1 : 0, is_f32(y), cur());
 }
 
-void gated_act(Tensor gu, int64_t F, int64_t kind, Tensor out) {
+void gated_act(Tensor gu, int64_t F, int64_t kind, Tensor out, double limit) {
   const c10::hip::OptionalHIPGuard g(dev_of(gu));
   TORCH_CHECK(gu.is_cuda() && act_ok(gu) && gu.dim() == 2 && gu.stride(1) == 1 && gu.size(1) >= 2 * F && F >= 1, "gu");
   CHECK_ACT(out, gu);
   TORCH_CHECK(out.is_contiguous() && out.dim() == 2 && out.size(0) == gu.size(0) && out.size(1) == F &&
-                  (kind == 0 || kind == 1), "out [T, F]");
-  sm_gated_act(gu.data_ptr(), gu.stride(0), F, kind, out.data_ptr(), gu.size(0), is_f32(gu), cur());
+                  kind >= 0 && kind <= 2, "out [T, F]");
+  sm_gated_act(gu.data_ptr(), gu.stride(0), F, kind, out.data_ptr(), gu.size(0), is_f32(gu), (float)limit, cur());
 }
 
 void qkv_rope_cache(Tensor qkv, std::optional<Tensor> bias, Tensor positions, std::optional<Tensor> cos_sin, int64_t Hq,
                     int64_t Hkv, int64_t dim, int64_t vdim, int64_t rot_dims, bool interleaved, bool unit, double eps,
-                    std::optional<Tensor> v_first, int64_t v_mode, double lam, Tensor slots, Tensor cache,
+                    std::optional<Tensor> v_first, int64_t v_mode, double lam, Tensor slots, std::optional<Tensor> cache_,
                     Tensor q_out, std::optional<Tensor> qk_w, bool norm_first, bool v_from_k,
                     std::optional<Tensor> conv_w, std::optional<Tensor> conv_state, std::optional<Tensor> row_seq,
                     std::optional<Tensor> seq_start, std::optional<Tensor> seq_slot, std::optional<Tensor> seq_init,
-                    int64_t max_q) {
+                    int64_t max_q, bool wide, std::optional<Tensor> q_scale) {
   const c10::hip::OptionalHIPGuard g(dev_of(qkv));
   TORCH_CHECK(qkv.is_cuda() && act_ok(qkv) && qkv.dim() == 2 && qkv.stride(1) == 1, "qkv");
   TORCH_CHECK(!v_from_k || (vdim == dim && v_mode == 0), "keys as values: vdim == dim, no value mixing");
   const int64_t T = qkv.size(0), n = (Hq + Hkv) * dim + (v_from_k ? 0 : Hkv * vdim);
-  TORCH_CHECK(Hq >= 1 && Hkv >= 1 && Hq % Hkv == 0 && dim >= 1 && dim <= 512 && vdim >= 1 && qkv.size(1) >= n, "sizes");
+  TORCH_CHECK(Hq >= 1 && Hkv >= 0 && dim >= 1 && dim <= 512 && vdim >= 1 && qkv.size(1) >= n, "sizes");
+  TORCH_CHECK(Hkv == 0 ? !cache_ && !v_from_k && v_mode == 0 && !conv_w : cache_ && Hq % Hkv == 0,
+              "queries only: no cache; otherwise whole groups of query heads");
   TORCH_CHECK(rot_dims >= 0 && rot_dims <= dim && rot_dims % 2 == 0, "rotary dims");
   TORCH_CHECK(positions.is_cuda() && positions.scalar_type() == torch::kInt64 && positions.is_contiguous() &&
                   positions.numel() == T && slots.is_cuda() && slots.scalar_type() == torch::kInt64 &&
@@ -433,9 +440,17 @@ void qkv_rope_cache(Tensor qkv, std::optional<Tensor> bias, Tensor positions, st
     CHECK_F32(*cos_sin);
     TORCH_CHECK(cos_sin->dim() == 2 && cos_sin->size(1) == rot_dims, "cos_sin [max_pos, rot_dims]");
   }
-  if (qk_w) {
+  if (wide) {
+    TORCH_CHECK(qk_w && !norm_first && !v_from_k && !conv_w, "norms over whole projections come with their weights alone");
+    CHECK_F32(*qk_w);
+    TORCH_CHECK(qk_w->numel() == (Hq + Hkv) * dim, "qk_w [q columns + k columns]");
+  } else if (qk_w) {
     CHECK_F32(*qk_w);
     TORCH_CHECK(unit && qk_w->numel() == 2 * dim, "qk_w [2, dim] goes with the unit norm");
+  }
+  if (q_scale) {
+    CHECK_F32(*q_scale);
+    TORCH_CHECK(q_scale->dim() == 1 && (!rot_dims || q_scale->size(0) == cos_sin->size(0)), "q_scale [max_pos]");
   }
   TORCH_CHECK(v_mode >= 0 && v_mode <= 2, "v_mode");
   if (v_mode) {
@@ -443,10 +458,12 @@ void qkv_rope_cache(Tensor qkv, std::optional<Tensor> bias, Tensor positions, st
     CHECK_F32(*v_first);
     TORCH_CHECK(v_first->numel() == T * Hkv * vdim, "v_first [T, Hkv * vdim]");
   }
-  CHECK_ACT(cache, qkv);
   CHECK_ACT(q_out, qkv);
-  TORCH_CHECK(cache.dim() == 4 && cache.is_contiguous() && cache.size(1) == Hkv && cache.size(3) == dim + vdim,
-              "cache [blocks, Hkv, bs, dim + vdim]");
+  if (cache_) {
+    CHECK_ACT(*cache_, qkv);
+    TORCH_CHECK(cache_->dim() == 4 && cache_->is_contiguous() && cache_->size(1) == Hkv && cache_->size(3) == dim + vdim,
+                "cache [blocks, Hkv, bs, dim + vdim]");
+  }
   TORCH_CHECK(q_out.is_contiguous() && q_out.numel() == T * Hq * dim, "q_out [T, Hq, dim]");
   int taps = 0;
   if (conv_w) {
@@ -464,13 +481,15 @@ void qkv_rope_cache(Tensor qkv, std::optional<Tensor> bias, Tensor positions, st
   }
   sm_qkv_rope_cache(qkv.data_ptr(), qkv.stride(0), bias ? bias->data_ptr<float>() : nullptr,
                     positions.data_ptr<int64_t>(), rot_dims ? cos_sin->data_ptr<float>() : nullptr, Hq, Hkv, dim, vdim,
-                    rot_dims, interleaved ? 1 : 0, unit ? 1 : 0, (float)eps, v_mode ? v_first->data_ptr<float>() : nullptr,
-                    v_mode, (float)lam, slots.data_ptr<int64_t>(), cache.data_ptr(), cache.size(2), q_out.data_ptr(),
+                    rot_dims, interleaved ? 1 : 0, unit && !wide ? 1 : 0, (float)eps, v_mode ? v_first->data_ptr<float>() : nullptr,
+                    v_mode, (float)lam, slots.data_ptr<int64_t>(), cache_ ? cache_->data_ptr() : nullptr,
+                    cache_ ? cache_->size(2) : 64, q_out.data_ptr(),
                     qk_w ? qk_w->data_ptr<float>() : nullptr, norm_first ? 1 : 0, v_from_k ? 1 : 0, T, is_f32(qkv),
                     taps ? conv_w->data_ptr() : nullptr, taps ? conv_state->data_ptr() : nullptr, taps,
                     taps ? row_seq->data_ptr<int>() : nullptr, taps ? seq_start->data_ptr<int>() : nullptr,
                     taps ? seq_slot->data_ptr<int>() : nullptr, taps ? seq_init->data_ptr<int>() : nullptr,
-                    taps ? seq_slot->numel() : 0, max_q, cur());
+                    taps ? seq_slot->numel() : 0, max_q, wide ? 1 : 0, q_scale ? q_scale->data_ptr<float>() : nullptr,
+                    cur());
 }
 
 void check_gqa(const Tensor& q, const Tensor& cache, int64_t dim, int64_t vdim, const Tensor& tables,
@@ -554,7 +573,8 @@ bool grouped_attention_mfma(Tensor q, Tensor cache, int64_t dim, int64_t vdim, T
   return rc == 0;
 }
 
-void moe_route_scores(Tensor logits, Tensor correction, int64_t k, Tensor ids, Tensor w) {
+void moe_route_scores(Tensor logits, Tensor correction, int64_t k, Tensor ids, Tensor w, int64_t groups, int64_t keep,
+                      double scale) {
   const c10::hip::OptionalHIPGuard g(dev_of(logits));
   CHECK_F32(logits);
   CHECK_F32(correction);
@@ -563,8 +583,10 @@ void moe_route_scores(Tensor logits, Tensor correction, int64_t k, Tensor ids, T
   const int T = logits.size(0), E = logits.size(1);
   TORCH_CHECK(logits.dim() == 2 && k >= 1 && k <= E && correction.numel() == E && ids.numel() == (int64_t)T * k &&
                   w.numel() == (int64_t)T * k, "router shapes");
+  TORCH_CHECK(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && k <= E / groups * keep,
+              "equal groups, enough of them kept");
   sm_moe_route_scores(logits.data_ptr<float>(), correction.data_ptr<float>(), E, k, ids.data_ptr<int>(),
-                      w.data_ptr<float>(), T, cur());
+                      w.data_ptr<float>(), T, groups, keep, (float)scale, cur());
 }
 
 void moe_route(Tensor logits, int64_t k, Tensor ids, Tensor w, bool sigmoid) {
@@ -593,7 +615,7 @@ void moe_group(Tensor ids, int64_t E, Tensor slot_row, Tensor tile_e, Tensor pai
 }
 
 void moe_gemm(Tensor A, int64_t kdiv, Tensor slot_row, Tensor tile_e, Tensor W, Tensor C, int64_t act, int64_t rows,
-              std::optional<Tensor> row_w) {
+              std::optional<Tensor> row_w, double limit) {
   const c10::hip::OptionalHIPGuard g(dev_of(A));
   TORCH_CHECK(A.is_cuda() && act_ok(A) && A.dim() == 2 && A.stride(1) == 1, "A");
   CHECK_ACT(W, A);
@@ -602,8 +624,8 @@ void moe_gemm(Tensor A, int64_t kdiv, Tensor slot_row, Tensor tile_e, Tensor W, 
   CHECK_I32(tile_e);
   TORCH_CHECK(W.dim() == 3 && W.is_contiguous() && W.size(2) == A.size(1), "W [E, N, K]");
   const int64_t mt = tile_e.numel();
-  const bool gated = act == 2 || act == 3;
-  TORCH_CHECK(act >= 0 && act <= 4 && (!gated || W.size(1) % 2 == 0), "epilogue");
+  const bool gated = act == 2 || act == 3 || act == 5;
+  TORCH_CHECK(act >= 0 && act <= 5 && (!gated || W.size(1) % 2 == 0), "epilogue");
   const int64_t N = gated ? W.size(1) / 2 : W.size(1);  // gated: W holds [gate rows | up rows]
   TORCH_CHECK(slot_row.numel() == mt * 64 && C.is_contiguous() && C.dim() == 2 && C.size(0) == mt * 64 &&
                   C.size(1) == N, "C [tiles * 64, N]");
@@ -614,7 +636,7 @@ void moe_gemm(Tensor A, int64_t kdiv, Tensor slot_row, Tensor tile_e, Tensor W, 
   }
   sm_moe_gemm(A.data_ptr(), A.stride(0), kdiv, slot_row.data_ptr<int>(), tile_e.data_ptr<int>(), W.data_ptr(),
               N, W.size(2), C.data_ptr(), mt, rows, (int)act, is_f32(A), row_w ? row_w->data_ptr<float>() : nullptr,
-              cur());
+              (float)limit, cur());
 }
 
 void moe_combine(Tensor y, Tensor pair_slot, std::optional<Tensor> w, Tensor out, std::optional<Tensor> h,
@@ -638,15 +660,16 @@ void moe_combine(Tensor y, Tensor pair_slot, std::optional<Tensor> w, Tensor out
     CHECK_ACT(*h, y);
     TORCH_CHECK(h->dim() == 2 && h->is_contiguous() && h->size(0) == T && h->size(1) == d, "h [T, d]");
   }
-  if (extra) {  // a shared expert's rows and their gate logits
+  if (extra) {  // a shared expert's rows and, unless they are added as they are, their gate logits
     CHECK_ACT(*extra, y);
     TORCH_CHECK(extra->dim() == 2 && extra->is_contiguous() && extra->size(0) == T && extra->size(1) == d, "extra [T, d]");
-    TORCH_CHECK(extra_gate && extra_gate->is_cuda() && extra_gate->scalar_type() == torch::kFloat32 &&
-                    extra_gate->dim() == 1 && extra_gate->size(0) == T, "extra_gate [T] fp32");
+    TORCH_CHECK(!extra_gate || (extra_gate->is_cuda() && extra_gate->scalar_type() == torch::kFloat32 &&
+                                extra_gate->dim() == 1 && extra_gate->size(0) == T), "extra_gate [T] fp32");
   }
   sm_moe_combine(y.data_ptr(), pair_slot.data_ptr<int>(), w ? w->data_ptr<float>() : nullptr, k, d, out.data_ptr(),
                  h ? h->data_ptr() : y.data_ptr(), T, is_f32(y), extra ? extra->data_ptr() : nullptr,
-                 extra ? extra_gate->data_ptr<float>() : nullptr, extra ? extra_gate->stride(0) : 0, cur());
+                 extra && extra_gate ? extra_gate->data_ptr<float>() : nullptr,
+                 extra && extra_gate ? extra_gate->stride(0) : 0, cur());
 }
 
 void bigram_embed(Tensor ids, Tensor table, double scale, std::optional<Tensor> bigram, int64_t buckets,
@@ -894,6 +917,59 @@ void hgrn2_scan(Tensor p, int64_t H, int64_t dk, int64_t dv, Tensor f_bias, Tens
   TORCH_CHECK(rc == 0, "hgrn2_scan: key size above 256");
 }
 
+// Retention over the projection p = [q | k | v (| g)]. The first nd sequences of the step bring one token each;
+// the runs of the others are cut into chunks by ``chunks``, the table of engine/attn_meta.py scan_chunks over
+// ALL sequences of the step: int32 [chunk bounds (nc + 1) | 3 nc numbers not used here | each sequence's first
+// chunk (nseq + 1)] (a sequence of one token is one chunk, so the chunks of the others start at number nd).
+void retention(Tensor p, int64_t H, int64_t dk, int64_t dv, bool gate, Tensor positions, std::optional<Tensor> cos_sin,
+               int64_t rot_dims, Tensor powers, double eps, Tensor state, Tensor seq_start, Tensor seq_slot,
+               Tensor seq_init, Tensor out, int64_t nd, std::optional<Tensor> chunks, int64_t nc) {
+  const c10::hip::OptionalHIPGuard g(dev_of(p));
+  TORCH_CHECK(H >= 1 && dk >= 1 && dv >= 1 && dk <= 4096 && dv <= 4096, "head count and sizes");
+  TORCH_CHECK(p.is_cuda() && act_ok(p) && p.dim() == 2 && p.stride(1) == 1 &&
+                  p.size(1) >= 2 * H * dk + (gate ? 2 : 1) * H * dv, "p [T, q | k | v (| g)]");
+  const int64_t T = p.size(0);
+  TORCH_CHECK(positions.is_cuda() && positions.scalar_type() == torch::kInt64 && positions.is_contiguous() &&
+                  positions.numel() == T, "positions: int64 [T]");
+  TORCH_CHECK(rot_dims >= 0 && rot_dims <= dk && rot_dims % 2 == 0, "rotary dims");
+  if (rot_dims) {
+    TORCH_CHECK(cos_sin.has_value(), "cos_sin");
+    CHECK_F32(*cos_sin);
+    TORCH_CHECK(cos_sin->dim() == 2 && cos_sin->size(1) == rot_dims, "cos_sin [max_pos, rot_dims]");
+  }
+  CHECK_F32(powers);
+  TORCH_CHECK(powers.dim() == 2 && powers.size(0) == H && powers.size(1) == sm_retention_chunk() + 1, "powers [H, chunk + 1]");
+  CHECK_F32(state);
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == dk && state.size(3) == dv,
+              "state [slots, H, dk, dv]");
+  check_seq(seq_start, seq_slot, seq_init, state.size(0));
+  const int64_t nseq = seq_slot.numel();
+  TORCH_CHECK(nseq <= 65535 && H <= 65535 && nd >= 0 && nd <= nseq, "too many sequences or heads in a step");
+  CHECK_ACT(out, p);
+  TORCH_CHECK(out.is_contiguous() && out.dim() == 2 && out.size(0) == T && out.size(1) == H * dv, "out [T, H dv]");
+  if (T == 0 || nseq == 0) return;
+  const int* ch = nullptr;
+  Tensor ws;
+  float *c_state = nullptr, *o_raw = nullptr;
+  if (nd < nseq) {
+    TORCH_CHECK(chunks.has_value(), "chunk table");
+    CHECK_I32(*chunks);
+    TORCH_CHECK(nc > nd && chunks->numel() == 4 * nc + 1 + nseq + 1, "chunk table");
+    ch = chunks->data_ptr<int>();
+    // fp32 workspaces: every chunk's state, and the read-outs when a head's columns take several workgroups
+    const int64_t n_cs = (nc - nd) * H * dk * dv, n_o = dv > sm_retention_cols() ? T * H * dv : 0;
+    ws = torch::empty({n_cs + n_o + 4}, torch::dtype(torch::kFloat32).device(p.device()));
+    c_state = ws.data_ptr<float>();
+    o_raw = n_o ? c_state + n_cs : nullptr;
+  }
+  const int rc = sm_retention(p.data_ptr(), p.stride(0), H, dk, dv, gate ? 1 : 0, positions.data_ptr<int64_t>(),
+                              rot_dims ? cos_sin->data_ptr<float>() : nullptr, rot_dims, powers.data_ptr<float>(),
+                              powers.size(1), (float)eps, state.data_ptr<float>(), seq_start.data_ptr<int>(),
+                              seq_slot.data_ptr<int>(), seq_init.data_ptr<int>(), out.data_ptr(), T, nseq, nd,
+                              is_f32(p), nc, ch, ch ? ch + 4 * nc + 1 : nullptr, c_state, o_raw, cur());
+  TORCH_CHECK(rc == 0, "retention: launch");
+}
+
 }  // namespace
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -931,4 +1007,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("hgrn2_scan", &hgrn2_scan);
   m.def("gated_add_norm", &gated_add_norm);
   m.def("poly_norm", &poly_norm);
+  m.def("retention", &retention);
 }

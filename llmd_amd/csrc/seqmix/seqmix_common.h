@@ -62,4 +62,11 @@ template <> struct Fn<uint16_t> {
 
 __device__ __forceinline__ float siluf_(float x) { return x / (1.f + expf(-x)); }
 
+// Clamped gated unit: g sigmoid(1.702 g) (v + 1), g cut off above ``limit``, v on both sides.
+__device__ __forceinline__ float clamped_unit(float g, float v, float limit) {
+  g = fminf(g, limit);
+  v = fminf(fmaxf(v, -limit), limit);
+  return g / (1.f + expf(-1.702f * g)) * (v + 1.f);
+}
+
 }  // namespace sm

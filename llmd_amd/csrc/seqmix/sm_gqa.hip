@@ -34,7 +34,10 @@
 // rotation; v_from_k - the values are the biased key projections themselves (no value columns); a
 // short convolution over time on every column of q, k and v, between the bias and everything else: a
 // token's earlier projections come from the step's own rows or from the sequence's state (its last
-// taps - 1 projected rows, stored without the bias), positions before 0 count as zeros.
+// taps - 1 projected rows, stored without the bias), positions before 0 count as zeros; wide - all q columns and
+// all k columns of a token are divided by their own root mean square and weighted (qk_w: one weight per column)
+// before the rotation, every workgroup of the token forming both sums; q_scale [max_pos] - the query at position
+// p is multiplied by q_scale[p]; Hkv 0 - the projection has queries only and nothing is cached.
 #include "seqmix_common.h"
 #include <algorithm>
 
@@ -62,7 +65,7 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_kernel(
     const float* __restrict__ cos_sin, int Hq, int Hkv, int dim, int vdim, int rot_dims, int interleaved, int unit,
     float eps, float* __restrict__ v_first, int v_mode, float lam, const int64_t* __restrict__ slots,
     T* __restrict__ cache, int bs, T* __restrict__ q_out, const float* __restrict__ qk_w, int norm_first,
-    int v_from_k, ConvArgs<T> cv) {
+    int v_from_k, ConvArgs<T> cv, int wide, const float* __restrict__ q_scale) {
   const int64_t t = blockIdx.x;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int half = rot_dims >> 1;
@@ -93,13 +96,29 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_kernel(
     }
     return a;
   };
+  float inv_q = 1.f, inv_k = 1.f;  // wide: of the whole projections
+  if (wide) {
+    __shared__ float red[NT / 64];
+    float sq = 0.f, sk = 0.f;
+    for (int e = threadIdx.x; e < Hq * dim; e += NT) {
+      const float x = val(e);
+      sq += x * x;
+    }
+    for (int e = threadIdx.x; e < Hkv * dim; e += NT) {
+      const float x = val(Hq * dim + e);
+      sk += x * x;
+    }
+    inv_q = 1.f / sqrtf(block_sum<NT>(sq, red) / (float)(Hq * dim) + eps);
+    if (Hkv > 0) inv_k = 1.f / sqrtf(block_sum<NT>(sk, red) / (float)(Hkv * dim) + eps);
+  }
+  if (q_scale) inv_q *= q_scale[pos];
   // blockIdx.y spreads a token's heads (a wave each) and value elements over workgroups: a step of
   // few tokens still fills the chip
   for (int hd = blockIdx.y * (NT / 64) + wave; hd < Hq + Hkv; hd += gridDim.y * (NT / 64)) {
     const bool is_q = hd < Hq;
     const int col0 = is_q ? hd * dim : Hq * dim + (hd - Hq) * dim;
-    const float* nw = qk_w ? qk_w + (is_q ? 0 : dim) : nullptr;  // the norm's weight, shared by the heads
-    const float* nw1 = norm_first ? nw : nullptr;               // applied before the rotation
+    const float* nw = qk_w ? qk_w + (wide ? col0 : is_q ? 0 : dim) : nullptr;  // the norm's weight
+    const float* nw1 = (norm_first || wide) ? nw : nullptr;                   // applied before the rotation
     float r[MAXE];
     float ss = 0.f;
 #pragma unroll
@@ -130,8 +149,8 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_kernel(
       r[i] = v;
       ss += norm_first ? raw * raw : v * v;
     }
-    float inv = 1.f;
-    if (unit) inv = 1.f / sqrtf(wave_sum(ss) / (float)dim + eps);
+    float inv = is_q ? inv_q : inv_k;
+    if (unit) inv *= 1.f / sqrtf(wave_sum(ss) / (float)dim + eps);
     T* dst = nullptr;
     if (is_q) dst = q_out + (t * Hq + hd) * dim;
     else if (slot >= 0) dst = cache + (blk * Hkv + (hd - Hq)) * bs * Dr + off * dim;
@@ -139,7 +158,7 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_kernel(
 #pragma unroll
     for (int i = 0; i < MAXE; ++i) {
       const int e = lane + 64 * i;
-      if (e < dim) st(dst + e, r[i] * inv * ((nw && !norm_first) ? nw[e] : 1.f));
+      if (e < dim) st(dst + e, r[i] * inv * ((nw && !nw1) ? nw[e] : 1.f));
     }
   }
   const int nv = Hkv * vdim, vcol0 = v_from_k ? Hq * dim : (Hq + Hkv) * dim;
@@ -195,7 +214,7 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_vec_kernel(
     int rot_dims, int interleaved, int unit, float eps, float* __restrict__ v_first, int v_mode, float lam,
     const int64_t* __restrict__ slots, bf16_t* __restrict__ cache, int bs, bf16_t* __restrict__ q_out,
     const float* __restrict__ qk_w, int norm_first, int v_from_k, ConvArgs<bf16_t> cv,
-    int gh, int tg, int T) {
+    int gh, int tg, int T, int wide, const float* __restrict__ q_scale) {
   if ((int)blockIdx.y >= gh) {
     const int nv = Hkv * vdim, vcol0 = v_from_k ? Hq * dim : (Hq + Hkv) * dim, nvb = (nv + NT - 1) / NT;
     const int unit = ((int)blockIdx.y - gh) * gridDim.x + blockIdx.x;
@@ -288,14 +307,31 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_vec_kernel(
   const int64_t blk = slot >= 0 ? slot / bs : 0, off = slot >= 0 ? slot % bs : 0;
   const int lph = dim >> 3, hpp = NT / lph;  // lanes per head, heads per pass
   const int c = threadIdx.x & (lph - 1), hl = threadIdx.x / lph;
+  float inv_q = 1.f, inv_k = 1.f;  // wide: of the whole projections
+  if (wide) {
+    __shared__ float red[NT / 64];
+    float sq = 0.f, sk = 0.f;
+    for (int e = threadIdx.x * 8; e < (Hq + Hkv) * dim; e += NT * 8) {  // a head is whole pieces of eight
+      float v[8], s8 = 0.f;
+      ld8(row + e, v);
+      if (bias) add8(bias + e, v);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) s8 += v[i] * v[i];
+      if (e < Hq * dim) sq += s8;
+      else sk += s8;
+    }
+    inv_q = 1.f / sqrtf(block_sum<NT>(sq, red) / (float)(Hq * dim) + eps);
+    if (Hkv > 0) inv_k = 1.f / sqrtf(block_sum<NT>(sk, red) / (float)(Hkv * dim) + eps);
+  }
+  if (q_scale) inv_q *= q_scale[pos];
   for (int h0 = blockIdx.y * hpp; h0 < Hq + Hkv; h0 += gh * hpp) {
     const int hd = h0 + hl;
     const bool on = hd < Hq + Hkv;
     const int col = hd * dim + c * 8;  // q heads, then k heads, back to back in the projection
     float x[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     float ss = 0.f;
-    const float* nw = qk_w ? qk_w + (hd < Hq ? 0 : dim) : nullptr;
-    const float* nw1 = norm_first ? nw : nullptr;  // weights applied before the rotation
+    const float* nw = qk_w ? qk_w + (wide ? hd * dim : hd < Hq ? 0 : dim) : nullptr;
+    const float* nw1 = (norm_first || wide) ? nw : nullptr;  // weights applied before the rotation
     if (on) {
       ld8(row + col, x);
       if (bias) add8(bias + col, x);
@@ -331,7 +367,7 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_vec_kernel(
               *reinterpret_cast<const uint4*>(row + col);
         }
       }
-      if (norm_first) {
+      if (norm_first || wide) {
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
           ss += x[i] * x[i];
@@ -378,17 +414,17 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_vec_kernel(
         }
       }
     }
-    float inv = 1.f;
+    float inv = hd < Hq ? inv_q : inv_k;
     if (unit) {
       if (!norm_first) {
 #pragma unroll
         for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
       }
       for (int o = lph >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);  // the head's lanes are an aligned group
-      inv = 1.f / sqrtf(ss / (float)dim + eps);
+      inv *= 1.f / sqrtf(ss / (float)dim + eps);
     }
     if (!on) continue;
-    if (nw && !norm_first) {
+    if (nw && !nw1) {
 #pragma unroll
       for (int i = 0; i < 8; ++i) x[i] *= nw[c * 8 + i];
     }
@@ -1173,7 +1209,8 @@ void sm_qkv_rope_cache(const void* qkv, int64_t stride, const float* bias, const
                        int unit, float eps, float* v_first, int v_mode, float lam, const int64_t* slots, void* cache,
                        int bs, void* q_out, const float* qk_w, int norm_first, int v_from_k, int T, int f32,
                        const void* conv_w, void* conv_state, int taps, const int* row_seq, const int* seq_start,
-                       const int* seq_slot, const int* seq_init, int nseq, int max_q, hipStream_t stream) {
+                       const int* seq_slot, const int* seq_init, int nseq, int max_q, int wide, const float* q_scale,
+                       hipStream_t stream) {
   if (T == 0) return;
   const int C = (Hq + Hkv) * dim + (v_from_k ? 0 : Hkv * vdim);
   const ConvArgs<float> cvf{(const float*)conv_w, (float*)conv_state, taps, C, row_seq, seq_start, seq_slot};
@@ -1185,7 +1222,7 @@ void sm_qkv_rope_cache(const void* qkv, int64_t stride, const float* bias, const
   if (f32)
     hipLaunchKernelGGL((qkv_rope_cache_kernel<float>), grid, dim3(NT), 0, stream, (const float*)qkv, stride, bias,
                        positions, cos_sin, Hq, Hkv, dim, vdim, rot_dims, interleaved, unit, eps, v_first, v_mode, lam,
-                       slots, (float*)cache, bs, (float*)q_out, qk_w, norm_first, v_from_k, cvf);
+                       slots, (float*)cache, bs, (float*)q_out, qk_w, norm_first, v_from_k, cvf, wide, q_scale);
   else if (dim % 8 == 0 && dim <= 512 && ((dim >> 3) & ((dim >> 3) - 1)) == 0 && stride % 8 == 0 &&
            rot_dims % (interleaved ? 8 : 16) == 0 && taps <= 8 && (taps == 0 || (C % 8 == 0 && !v_from_k)) &&
            (((uintptr_t)qkv | (uintptr_t)q_out | (uintptr_t)cache | (uintptr_t)bias | (uintptr_t)cos_sin |
@@ -1200,7 +1237,8 @@ void sm_qkv_rope_cache(const void* qkv, int64_t stride, const float* bias, const
   case N:                                                                                                             \
     hipLaunchKernelGGL(qkv_rope_cache_vec_kernel<N>, vgrid, dim3(NT), 0, stream, (const bf16_t*)qkv, stride, bias,    \
                        positions, cos_sin, Hq, Hkv, dim, vdim, rot_dims, interleaved, unit, eps, v_first, v_mode, lam, \
-                       slots, (bf16_t*)cache, bs, (bf16_t*)q_out, qk_w, norm_first, v_from_k, cvh, gh, tg, T);        \
+                       slots, (bf16_t*)cache, bs, (bf16_t*)q_out, qk_w, norm_first, v_from_k, cvh, gh, tg, T, wide,   \
+                       q_scale);                                                                                      \
     break
     switch (taps) {
       SM_QRC(0); SM_QRC(1); SM_QRC(2); SM_QRC(3); SM_QRC(4); SM_QRC(5); SM_QRC(6); SM_QRC(7); SM_QRC(8);
@@ -1212,7 +1250,7 @@ void sm_qkv_rope_cache(const void* qkv, int64_t stride, const float* bias, const
   } else
     hipLaunchKernelGGL((qkv_rope_cache_kernel<bf16_t>), grid, dim3(NT), 0, stream, (const bf16_t*)qkv, stride, bias,
                        positions, cos_sin, Hq, Hkv, dim, vdim, rot_dims, interleaved, unit, eps, v_first, v_mode, lam,
-                       slots, (bf16_t*)cache, bs, (bf16_t*)q_out, qk_w, norm_first, v_from_k, cvh);
+                       slots, (bf16_t*)cache, bs, (bf16_t*)q_out, qk_w, norm_first, v_from_k, cvh, wide, q_scale);
   sm_conv_state(qkv, stride, C, taps, conv_state, seq_start, seq_slot, seq_init, nseq, 0, f32, stream);
 }
 

@@ -2,8 +2,10 @@
 // W_down (act(W_gate h) * (W_up h)) with [gate rows | up rows] stacked in one weight per expert.
 //
 // moe_route_scores : softmax over all router outputs, the k largest of score + correction chosen,
-//               weights = chosen scores / (their sum + 1e-20).
-// epilogues of moe_gemm (ACT): 0 none, 1 erf-GELU, 2 tanh-GELU(gate) * up, 3 SiLU(gate) * up, 4 squared ReLU. In the
+//               weights = chosen scores / (their sum + 1e-20) * scale. With groups the outputs form equal groups of
+//               neighbours and only those of the best ``keep`` groups (by their largest score + correction) count.
+// epilogues of moe_gemm (ACT): 0 none, 1 erf-GELU, 2 tanh-GELU(gate) * up, 3 SiLU(gate) * up, 4 squared ReLU,
+//               5 clamped units of gate and up (seqmix_common.h). In the
 //               gated forms a workgroup's B tile holds matching gate and up columns, so the product is
 //               formed in registers and only F columns are written.
 // ids >= E (identity experts) get no tile: moe_group marks their pairs -1 and moe_combine adds
@@ -15,7 +17,8 @@
 // moe_gemm    : tile GEMM, 64 rows x 64 columns per workgroup, K stepped by 16 through LDS,
 //               4 x 4 outputs per thread, fp32 accumulation in a fixed K order (a row's sums do
 //               not depend on its tile or on the rest of the step); optional erf-GELU epilogue.
-// moe_combine : out[t] = sum_j w[t, j] * y[slot(t, j)] (+ sigmoid(g[t]) * extra[t], a shared expert's row) in fp32.
+// moe_combine : out[t] = sum_j w[t, j] * y[slot(t, j)] (+ extra[t], a shared expert's row, times sigmoid(g[t]) when it
+//               has a gate) in fp32.
 #include "seqmix_common.h"
 
 using namespace sm;
@@ -118,7 +121,7 @@ __global__ __launch_bounds__(256) void moe_route_wave_kernel(const float* __rest
 __global__ __launch_bounds__(256) void moe_route_scores_wave_kernel(const float* __restrict__ logits,
                                                                     const float* __restrict__ corr, int E, int k,
                                                                     int* __restrict__ ids, float* __restrict__ w,
-                                                                    int T) {
+                                                                    int T, int groups, int keep, float scale) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
   const int lane = threadIdx.x & 63;
   if (t >= T) return;
@@ -144,6 +147,32 @@ __global__ __launch_bounds__(256) void moe_route_scores_wave_kernel(const float*
     const int e = lane + 64 * i;
     sc[i] = sc[i] / sum;                            // the score
     v[i] = e < E ? sc[i] + corr[e] : -INFINITY;     // what the choice looks at
+  }
+  if (groups > 1) {  // groups <= 64: lane g keeps the largest choice score of group g
+    const int per = E / groups;
+    float gbest = -INFINITY;
+    for (int g = 0; g < groups; ++g) {
+      float m = -INFINITY;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int e = lane + 64 * i;
+        if (e >= g * per && e < (g + 1) * per) m = fmaxf(m, v[i]);
+      }
+      m = wave_max(m);
+      if (lane == g) gbest = m;
+    }
+    // a group's rank: how many are larger, or equal with a lower index
+    int rank = 0;
+    for (int g = 0; g < groups; ++g) {
+      const float o = __shfl(gbest, g, 64);
+      rank += (o > gbest || (o == gbest && g < lane)) ? 1 : 0;
+    }
+    const uint64_t kept = __ballot(lane < groups && rank < keep);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const int e = lane + 64 * i;
+      if (e < E && !(kept >> (e / per) & 1ull)) v[i] = -INFINITY;
+    }
   }
   float wsum = 0.f, mine = 0.f;
   int mine_id = 0;
@@ -179,14 +208,15 @@ __global__ __launch_bounds__(256) void moe_route_scores_wave_kernel(const float*
   }
   if (lane < k) {
     ids[(int64_t)t * k + lane] = mine_id;
-    w[(int64_t)t * k + lane] = mine / (wsum + 1e-20f);
+    w[(int64_t)t * k + lane] = mine / (wsum + 1e-20f) * scale;
   }
 }
 
 // Any E: one thread per token.
 __global__ __launch_bounds__(256) void moe_route_scores_kernel(const float* __restrict__ logits,
                                                                const float* __restrict__ corr, int E, int k,
-                                                               int* __restrict__ ids, float* __restrict__ w, int T) {
+                                                               int* __restrict__ ids, float* __restrict__ w, int T,
+                                                               int groups, int keep, float scale) {
   const int t = blockIdx.x * 256 + threadIdx.x;
   if (t >= T) return;
   const float* z = logits + (int64_t)t * E;
@@ -195,11 +225,43 @@ __global__ __launch_bounds__(256) void moe_route_scores_kernel(const float* __re
   float mx = -INFINITY, sum = 0.f;
   for (int e = 0; e < E; ++e) mx = fmaxf(mx, z[e]);
   for (int e = 0; e < E; ++e) sum += expf(z[e] - mx);
+  const int per = E / groups;
+  auto group_best = [&](int g) {
+    float m = -INFINITY;
+    for (int e = g * per; e < (g + 1) * per; ++e) m = fmaxf(m, expf(z[e] - mx) / sum + corr[e]);
+    return m;
+  };
+  // the last group kept: one after the other in falling order, ties to the lower index
+  float last = INFINITY;
+  int last_g = -1;
+  if (groups > 1) {
+    for (int n = 0; n < keep; ++n) {
+      float best = -INFINITY;
+      int bg = -1;
+      for (int g = 0; g < groups; ++g) {
+        const float m = group_best(g);
+        const bool after = m < last || (m == last && g > last_g);
+        if (after && (bg < 0 || m > best)) {
+          best = m;
+          bg = g;
+        }
+      }
+      last = best;
+      last_g = bg;
+    }
+  }
   float wsum = 0.f;
   for (int j = 0; j < k; ++j) {
     float best = -INFINITY, bsc = 0.f;
     int bi = -1;
     for (int e = 0; e < E; ++e) {
+      if (groups > 1 && e % per == 0) {
+        const float m = group_best(e / per);
+        if (m < last || (m == last && e / per > last_g)) {  // not kept
+          e += per - 1;
+          continue;
+        }
+      }
       bool taken = false;
       for (int i = 0; i < j; ++i) taken |= oi[i] == e;
       const float sc = expf(z[e] - mx) / sum;
@@ -214,7 +276,7 @@ __global__ __launch_bounds__(256) void moe_route_scores_kernel(const float* __re
     ow[j] = bsc;
     wsum += bsc;
   }
-  for (int j = 0; j < k; ++j) ow[j] /= (wsum + 1e-20f);
+  for (int j = 0; j < k; ++j) ow[j] = ow[j] / (wsum + 1e-20f) * scale;
 }
 
 __global__ __launch_bounds__(1024) void moe_group_kernel(const int* __restrict__ ids, int n, int E,
@@ -259,12 +321,14 @@ __device__ __forceinline__ float gelu_erf_(float v) { return 0.5f * v * (1.f + e
 __device__ __forceinline__ float gelu_tanh_(float v) {
   return 0.5f * v * (1.f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
 }
+constexpr bool gated_act_code(int act) { return act == 2 || act == 3 || act == 5; }
 template <int ACT>
-__device__ __forceinline__ float gate_act_(float g) {
-  return ACT == 2 ? gelu_tanh_(g) : g / (1.f + expf(-g));
+__device__ __forceinline__ float gated_(float g, float u, float limit) {
+  if (ACT == 5) return clamped_unit(g, u, limit);
+  return (ACT == 2 ? gelu_tanh_(g) : g / (1.f + expf(-g))) * u;
 }
 
-// Gated forms (ACT 2 and 3): N is the number of OUTPUT columns F; the weight has 2 N rows [gate | up].
+// Gated forms (ACT 2, 3 and 5): N is the number of OUTPUT columns F; the weight has 2 N rows [gate | up].
 // The workgroup's 64 B rows are 32 gate rows n0.. and the 32 matching up rows; a thread's four
 // columns are two gate columns and their two up columns.
 template <typename T, int ACT>
@@ -272,14 +336,14 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ A, 
                                                        const int* __restrict__ slot_row,
                                                        const int* __restrict__ tile_e, const T* __restrict__ Wt,
                                                        int N, int K, T* __restrict__ Cout,
-                                                       const float* __restrict__ row_w) {
+                                                       const float* __restrict__ row_w, float limit) {
   const int e = tile_e[blockIdx.x];
   if (e < 0) return;
   __shared__ float sA[TK][TM + 4], sB[TK][TN + 4];
   __shared__ int srow[TM];
   __shared__ float sw[TM];  // the row's input weight (gated forms with row_w): scales both sums
   const int tid = threadIdx.x;
-  constexpr bool GATED = ACT == 2 || ACT == 3;
+  constexpr bool GATED = gated_act_code(ACT);
   const int slot0 = blockIdx.x * TM, n0 = blockIdx.y * (GATED ? TN / 2 : TN);
   if (tid < TM) {
     const int p = slot_row[slot0 + tid];
@@ -325,7 +389,7 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ A, 
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         const int n = n0 + tx * 2 + j;
-        if (n < N) st(Cout + (int64_t)(slot0 + r) * N + n, gate_act_<ACT>(sw[r] * acc[i][j]) * (sw[r] * acc[i][j + 2]));
+        if (n < N) st(Cout + (int64_t)(slot0 + r) * N + n, gated_<ACT>(sw[r] * acc[i][j], sw[r] * acc[i][j + 2], limit));
       }
       continue;
     }
@@ -358,7 +422,7 @@ constexpr int MBK = 64, MLS = MBK + 8;  // LDS row stride 144 B
 // NJ = 16-column fragments per wave: the workgroup's tile is 64 rows x MBN = 32 NJ columns
 // (128 for steps with few rows per expert: more workgroups stream the weights; 256 for prompt-sized
 // steps: twice the MFMAs per LDS pass and barrier).
-// Gated forms (ACT 2 and 3): a wave's first NJ / 2 fragments are gate columns, the other NJ / 2 the
+// Gated forms (ACT 2, 3 and 5): a wave's first NJ / 2 fragments are gate columns, the other NJ / 2 the
 // matching up columns; the workgroup writes 16 NJ output columns.
 template <int ACT, int NJ>
 __global__ __launch_bounds__(256) void moe_gemm_mfma_kernel(const bf16_t* __restrict__ A, int64_t a_stride, int kdiv,
@@ -366,10 +430,10 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_kernel(const bf16_t* __rest
                                                             const int* __restrict__ tile_e,
                                                             const bf16_t* __restrict__ Wt, int N, int K,
                                                             bf16_t* __restrict__ Cout,
-                                                            const float* __restrict__ row_w) {
+                                                            const float* __restrict__ row_w, float limit) {
   const int e = tile_e[blockIdx.x];
   if (e < 0) return;
-  constexpr bool GATED = ACT == 2 || ACT == 3;
+  constexpr bool GATED = gated_act_code(ACT);
   constexpr int MBN = 32 * NJ, NB = MBN / 32;  // NB = B chunks per thread and K step
   __shared__ __attribute__((aligned(16))) bf16_t sA[TM * MLS];
   __shared__ __attribute__((aligned(16))) bf16_t sB[MBN * MLS];
@@ -465,7 +529,7 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_kernel(const bf16_t* __rest
           const int n = n0 + wn * 8 * NJ + j * 16 + r16;
           if (n < N)
             st(Cout + (int64_t)(slot0 + row) * N + n,
-               gate_act_<ACT>(sw[row] * acc[i][j][r]) * (sw[row] * acc[i][j + NJ / 2][r]));
+               gated_<ACT>(sw[row] * acc[i][j][r], sw[row] * acc[i][j + NJ / 2][r], limit));
         }
         continue;
       }
@@ -491,7 +555,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const T* __restrict__ 
                                                           const T* __restrict__ extra,
                                                           const float* __restrict__ eg, int64_t eg_stride) {
   const int64_t t = blockIdx.x;
-  const float ge = extra ? 1.f / (1.f + expf(-eg[t * eg_stride])) : 0.f;
+  const float ge = eg ? 1.f / (1.f + expf(-eg[t * eg_stride])) : 1.f;
   for (int c = threadIdx.x; c < d; c += 256) {
     float s = 0.f;
     for (int j = 0; j < k; ++j) {
@@ -512,7 +576,7 @@ __global__ __launch_bounds__(256) void moe_combine_vec_kernel(const bf16_t* __re
                                                               const bf16_t* __restrict__ extra,
                                                               const float* __restrict__ eg, int64_t eg_stride) {
   const int64_t t = blockIdx.x;
-  const float ge = extra ? 1.f / (1.f + expf(-eg[t * eg_stride])) : 0.f;
+  const float ge = eg ? 1.f / (1.f + expf(-eg[t * eg_stride])) : 1.f;
   for (int c = threadIdx.x * 8; c < d; c += 256 * 8) {
     float s[8] = {};
     for (int j = 0; j < k; ++j) {
@@ -555,16 +619,16 @@ void sm_moe_route(const float* logits, int64_t stride, int E, int k, int* ids, f
                      sigmoid);
 }
 
-void sm_moe_route_scores(const float* logits, const float* corr, int E, int k, int* ids, float* w, int T,
-                         hipStream_t stream) {
+void sm_moe_route_scores(const float* logits, const float* corr, int E, int k, int* ids, float* w, int T, int groups,
+                         int keep, float scale, hipStream_t stream) {
   if (T == 0) return;
-  if (E <= 512 && k <= 64) {
+  if (E <= 512 && k <= 64 && groups <= 64) {
     hipLaunchKernelGGL(moe_route_scores_wave_kernel, dim3((T + 3) / 4), dim3(256), 0, stream, logits, corr, E, k, ids,
-                       w, T);
+                       w, T, groups, keep, scale);
     return;
   }
   hipLaunchKernelGGL(moe_route_scores_kernel, dim3((T + 255) / 256), dim3(256), 0, stream, logits, corr, E, k, ids, w,
-                     T);
+                     T, groups, keep, scale);
 }
 
 void sm_moe_group(const int* ids, int n, int E, int* slot_row, int* tile_e, int* pair_slot, int max_tiles,
@@ -573,14 +637,14 @@ void sm_moe_group(const int* ids, int n, int E, int* slot_row, int* tile_e, int*
                      pair_slot, max_tiles);
 }
 
-// act: 0 none, 1 erf-GELU, 2 tanh-GELU(gate) * up, 3 SiLU(gate) * up, 4 squared ReLU. N = output columns (the gated
-// forms read a weight of 2 N rows per expert).
+// act: 0 none, 1 erf-GELU, 2 tanh-GELU(gate) * up, 3 SiLU(gate) * up, 4 squared ReLU, 5 clamped units. N = output
+// columns (the gated forms read a weight of 2 N rows per expert).
 // row_w (gated forms): fp32 weight per (token, choice) pair that scales the row's INPUT, applied to
 // both fp32 sums before the activation; nullptr = 1.
 void sm_moe_gemm(const void* A, int64_t a_stride, int kdiv, const int* slot_row, const int* tile_e, const void* W,
-                 int N, int K, void* C, int max_tiles, int rows_hint, int act, int f32, const float* row_w,
+                 int N, int K, void* C, int max_tiles, int rows_hint, int act, int f32, const float* row_w, float limit,
                  hipStream_t stream) {
-  const bool gated = act == 2 || act == 3;
+  const bool gated = gated_act_code(act);
   if (!f32 && K % 8 == 0 && a_stride % 8 == 0 && ((uintptr_t)A & 15) == 0 && ((uintptr_t)W & 15) == 0) {
     // wide tiles when the step has prompt-sized row counts (most tiles are full) and N is wide
     const bool wide = N >= 256 && rows_hint >= 32 * max_tiles;
@@ -588,7 +652,7 @@ void sm_moe_gemm(const void* A, int64_t a_stride, int kdiv, const int* slot_row,
     const dim3 g2(max_tiles, (N + mbn - 1) / mbn);
 #define SM_MF(A_, NJ)                                                                                          \
   hipLaunchKernelGGL((moe_gemm_mfma_kernel<A_, NJ>), g2, dim3(256), 0, stream, (const bf16_t*)A, a_stride, kdiv, \
-                     slot_row, tile_e, (const bf16_t*)W, N, K, (bf16_t*)C, row_w)
+                     slot_row, tile_e, (const bf16_t*)W, N, K, (bf16_t*)C, row_w, limit)
 #define SM_MF2(A_) \
   if (wide) SM_MF(A_, 8); \
   else SM_MF(A_, 4)
@@ -596,7 +660,8 @@ void sm_moe_gemm(const void* A, int64_t a_stride, int kdiv, const int* slot_row,
     else if (act == 1) { SM_MF2(1); }
     else if (act == 2) { SM_MF2(2); }
     else if (act == 3) { SM_MF2(3); }
-    else { SM_MF2(4); }
+    else if (act == 4) { SM_MF2(4); }
+    else { SM_MF2(5); }
 #undef SM_MF2
 #undef SM_MF
     return;
@@ -605,20 +670,21 @@ void sm_moe_gemm(const void* A, int64_t a_stride, int kdiv, const int* slot_row,
   const dim3 grid(max_tiles, (N + tn - 1) / tn);
 #define SM_GO(TYPE, A_)                                                                                         \
   hipLaunchKernelGGL((moe_gemm_kernel<TYPE, A_>), grid, dim3(256), 0, stream, (const TYPE*)A, a_stride, kdiv,   \
-                     slot_row, tile_e, (const TYPE*)W, N, K, (TYPE*)C, row_w)
+                     slot_row, tile_e, (const TYPE*)W, N, K, (TYPE*)C, row_w, limit)
 #define SM_GO2(TYPE)                   \
   if (act == 0) SM_GO(TYPE, 0);        \
   else if (act == 1) SM_GO(TYPE, 1);   \
   else if (act == 2) SM_GO(TYPE, 2);   \
   else if (act == 3) SM_GO(TYPE, 3);   \
-  else SM_GO(TYPE, 4)
+  else if (act == 4) SM_GO(TYPE, 4);   \
+  else SM_GO(TYPE, 5)
   if (f32) { SM_GO2(float); }
   else { SM_GO2(bf16_t); }
 #undef SM_GO2
 #undef SM_GO
 }
 
-// extra [T, d] with its gate logits eg (fp32, row stride eg_stride): a shared expert's rows, or null.
+// extra [T, d] with its gate logits eg (fp32, row stride eg_stride; null: no gate): a shared expert's rows, or null.
 void sm_moe_combine(const void* y, const int* pair_slot, const float* w, int k, int d, void* out, const void* h, int T,
                     int f32, const void* extra, const float* eg, int64_t eg_stride, hipStream_t stream) {
   if (T == 0) return;

@@ -72,7 +72,7 @@ class ModelConfig:
     layer_specs: Optional[list] = None
     embedding_scale: float = 1.0
     logit_softcap: float = 0.0
-    # hyper-connections (models/negunex.py): number of residual streams, 0 = one plain residual
+    # hyper-connections (models/hyper.py): number of residual streams, 0 = one plain residual
     hyper_streams: int = 0
     # hashed bigram table added to the embedding (models/zumizen.py): {buckets, mul_prev, mul_cur} or None
     bigram: Optional[dict] = None
@@ -130,6 +130,8 @@ class ModelConfig:
             return kakalorn_config(d)
         if d.get("architecture") == "Kokatar":
             return kokatar_config(d)
+        if d.get("architecture") == "Koduzen":
+            return koduzen_config(d)
         names = {f.name for f in dataclasses.fields(cls)}
         kw = {k: v for k, v in d.items() if k in names}
         if "num_experts" in d and "num_local_experts" not in d:
@@ -301,6 +303,53 @@ def kokatar_config(d: dict) -> ModelConfig:
         rms_norm_eps=d["norm"]["eps"], max_position_embeddings=d.get("max_position", 1 << 20),
         bos_token_id=d.get("bos", 0), eos_token_id=d.get("eos", -1), layer_specs=layers,
         conv_taps=int((d.get("canon") or {}).get("taps", 1)), name=d.get("name", "kokatar"))
+
+
+KODUZEN_MIXERS = ("attention", "attention_2", "retention")
+
+
+def koduzen_config(d: dict) -> ModelConfig:
+    """A Koduzen ``config.json``: ``layers`` lists every layer (``type`` "attention", "attention_2" or
+    "retention", the ``mixer``'s sizes and constants, ``mlp`` - dense or experts with a shared one - or
+    null), ``streams`` the residual streams joined by hyper-connections, ``norm.eps``, ``vocab``, ``width``.
+    The head is the embedding table. An attention layer with ``kv_from`` reads the keys and values of an
+    earlier one of its kind, which must have projections of its own and the same key/value heads, sizes
+    and rotation."""
+    layers = [json.loads(json.dumps(l)) for l in d["layers"]]
+    for i, l in enumerate(layers):
+        m, f = l["mixer"], l.get("mlp")
+        if l["type"] not in KODUZEN_MIXERS:
+            raise ValueError(f"koduzen: layer {i} has the unknown mixer type {l['type']!r}")
+        src = m.get("kv_from")
+        if src is not None:
+            ok = l["type"] != "retention" and 0 <= src < i and layers[src]["type"] == l["type"] and \
+                layers[src]["mixer"].get("kv_from") is None
+            if not ok or any(layers[src]["mixer"].get(k) != m.get(k) for k in ("kv_heads", "dim", "vdim", "rot")):
+                raise ValueError(f"koduzen: layer {i} cannot read the keys and values of layer {src}")
+        if l["type"] == "retention" and len(m["decay"]) != m["heads"]:
+            raise ValueError(f"koduzen: layer {i} has {m['heads']} heads and {len(m['decay'])} decays")
+        if f and f["kind"] not in ("dense", "moe"):
+            raise ValueError(f"koduzen: layer {i} has the unknown feed-forward kind {f['kind']!r}")
+        if f and f["kind"] == "moe":
+            r = f["router"]
+            n, g = r["experts"] + r.get("identity", 0), r.get("groups") or {"count": 1, "keep": 1}
+            if n % g["count"] or not 1 <= g["keep"] <= g["count"] or r["top"] > n // g["count"] * g["keep"]:
+                raise ValueError(f"koduzen: layer {i} cannot choose {r['top']} of {n} experts in {g['count']} groups, "
+                                 f"{g['keep']} of them kept")
+    att = [l["mixer"] for l in layers if l["type"] != "retention"]
+    mlps = [l["mlp"] for l in layers if l.get("mlp")]
+    moe = [m for m in mlps if m["kind"] == "moe"]
+    return ModelConfig(
+        model_type="koduzen", hidden_size=d["width"], vocab_size=d["vocab"], num_hidden_layers=len(layers),
+        num_attention_heads=att[0]["heads"] if att else 1, num_key_value_heads=att[0]["kv_heads"] if att else 1,
+        head_dim=att[0]["dim"] if att else 1, v_head_dim=att[0]["vdim"] if att else 0,
+        intermediate_size=max([m["ff"] for m in mlps if m["kind"] == "dense"] or [0]),
+        num_local_experts=max([m["router"]["experts"] for m in moe] or [0]),
+        num_experts_per_tok=max([m["router"]["top"] for m in moe] or [0]),
+        moe_intermediate_size=max([m["expert"]["ff"] for m in moe] or [0]),
+        rms_norm_eps=d["norm"]["eps"], max_position_embeddings=d.get("max_position", 1 << 20),
+        bos_token_id=d.get("bos", 0), eos_token_id=d.get("eos", -1), layer_specs=layers, tie_word_embeddings=True,
+        hyper_streams=int(d.get("streams") or 0), name=d.get("name", "koduzen"))
 
 
 def _llama(name, d, ffn, L, hq, hkv, vocab=128256, **kw):
@@ -520,6 +569,30 @@ def _tiny_kokatar() -> ModelConfig:
 
 
 _register(_tiny_kokatar())
+
+
+def _tiny_koduzen() -> ModelConfig:
+    """Random-weight preset with all three mixer kinds, a layer that shares keys and values, both
+    feed-forward kinds and a layer without one."""
+    rot = {"dims": 16, "base": 10000.0}
+    att = {"heads": 4, "kv_heads": 2, "dim": 32, "vdim": 16, "scale": 32 ** -0.5, "mask": {"size": 24},
+           "rot": dict(rot, scaling={"factor": 4.0, "original": 64, "fast": 8.0, "slow": 1.0})}
+    att2 = {"heads": 4, "kv_heads": 1, "dim": 16, "vdim": 24, "scale": 0.25, "mask": {"size": 40},
+            "q_temp": {"coef": 0.3, "every": 16}}
+    ret = {"heads": 3, "dim": 16, "vdim": 32, "rot": rot, "decay": [0.9, 0.97, 0.995]}
+    dense = {"kind": "dense", "ff": 192, "limit": 2.0}
+    moe = {"kind": "moe", "expert": {"ff": 48, "limit": 1.5}, "shared": {"ff": 64, "limit": 3.0},
+           "router": {"experts": 6, "identity": 2, "top": 2, "groups": {"count": 4, "keep": 2}, "scale": 1.25}}
+    return koduzen_config({
+        "architecture": "Koduzen", "name": "tiny-koduzen", "width": 128, "vocab": 512, "norm": {"eps": 1e-6}, "streams": 2,
+        "max_position": 4096, "eos": 1,
+        "layers": [{"type": "retention", "mixer": ret, "mlp": moe},
+                   {"type": "attention_2", "mixer": att2, "mlp": dense},
+                   {"type": "attention", "mixer": att, "mlp": None},
+                   {"type": "attention_2", "mixer": dict(att2, kv_from=1), "mlp": moe}]})
+
+
+_register(_tiny_koduzen())
 
 
 def get_model_config(name_or_path: str) -> ModelConfig:

@@ -52,6 +52,10 @@ def model_class(cfg: ModelConfig):
         from .kokatar import KokatarForCausalLM
 
         return KokatarForCausalLM
+    if t == "koduzen":
+        from .koduzen import KoduzenForCausalLM
+
+        return KoduzenForCausalLM
     raise ValueError(f"unsupported model_type {t!r}")
 
 

@@ -33,6 +33,11 @@ constant is an argument, so another stack can reuse them.
 * ``SharedMoE``        - ungated squared-ReLU experts, softmax over the chosen logits, beside a shared expert
   behind a sigmoid.
 * ``ResidualGates``    - sigmoid(W h + b) for every sublayer of a layer, multiplied with its result.
+* ``GroupedAttention`` options: norms over whole projections, queries warmed with their position, the keys and
+  values of an earlier layer's cache instead of its own.
+* ``RetentionMixer``   - linear attention with a fixed decay per head.
+* ``GatedMLP`` / ``ScoreMoE`` options: clamped gated units, experts chosen inside the best groups, a scale on
+  the weights, a shared expert for every token.
 
 Recurrent state lives in the engine's state pool (engine/state_cache.py): a mixer with
 ``state_shapes()`` gets its per-slot tensors through ``bind_state``; the step's
@@ -332,12 +337,18 @@ class GroupedAttention(torch.nn.Module):
     conv         > 0: a causal convolution over time with that many taps on every column of the biased
                  projections q, k and v (``conv``), ahead of everything else; its state is the
                  sequence's last conv - 1 projected rows (``self.conv``, a state layer)
+    wide_norm    RMS norms over ALL rows of q and of k, before they are split into heads and rotated, with
+                 weights ``q_norm`` / ``k_norm`` of those sizes
+    q_temp       {coef, every}: the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1)
+    kv_source    an earlier GroupedAttention whose cached keys and values this layer reads instead of projecting
+                 and writing its own (no k and v rows here; queries, mask and everything else are this layer's)
     """
     is_latent = False
 
     def __init__(self, d_model, heads, kv_heads, dim, vdim, scale, rot, eps, max_pos, device, dtype, bias=True,
                  interleaved=True, unit_norm=True, v_mix=False, gate=True, norm_weight=False, slopes=None, chunk=0,
-                 sink=False, out_bias=False, v_from_k=False, norm_first=False, window=0, keep_first=0, conv=0):
+                 sink=False, out_bias=False, v_from_k=False, norm_first=False, window=0, keep_first=0, conv=0,
+                 wide_norm=False, q_temp=None, kv_source=None):
         super().__init__()
         if heads % kv_heads:
             raise ValueError(f"{heads} query heads do not divide over {kv_heads} key/value heads")
@@ -345,12 +356,22 @@ class GroupedAttention(torch.nn.Module):
             raise ValueError("values that are the keys need vdim == dim and no value mixing")
         if window and chunk:
             raise ValueError("a sliding window and chunks do not combine")
+        if wide_norm and (unit_norm or conv or v_from_k):
+            raise ValueError("norms over whole projections do not combine with unit norms, a convolution or keys as values")
+        self._src = [kv_source] if kv_source is not None else None   # a list: not a submodule of this layer
+        if kv_source is not None:
+            if v_mix or v_from_k or conv:
+                raise ValueError("shared keys and values do not combine with value mixing, keys as values or a convolution")
+            if (kv_source.Hkv, kv_source.dim, kv_source.vdim, kv_source._src) != (kv_heads, dim, vdim, None):
+                raise ValueError("shared keys and values need the same kv heads and sizes and a layer that owns them")
         self.Hq, self.Hkv, self.dim, self.vdim = heads, kv_heads, dim, vdim
         self.scale, self.eps, self.interleaved, self.unit_norm = float(scale), eps, interleaved, unit_norm
         self.v_mix, self.has_gate = bool(v_mix), bool(gate)
         self.v_from_k, self.norm_first = bool(v_from_k), bool(norm_first)
         self.win, self.keep_first = int(window), int(keep_first) if window else 0
         self.nq, self.nk, self.nv = heads * dim, kv_heads * dim, 0 if v_from_k else kv_heads * vdim
+        if kv_source is not None:
+            self.nk = self.nv = 0
         n = self.nq + self.nk + self.nv + (heads * vdim if gate else 0)
         self.n_out = -(-n // 8) * 8  # rows of 16-byte multiples for the vector loads downstream
         self.proj = ColumnLinear(d_model, self.n_out, shard=False, device=device, dtype=dtype)
@@ -365,6 +386,15 @@ class GroupedAttention(torch.nn.Module):
                 raise ValueError("norm weights need the unit norm")
             self.q_norm = _param((dim,), device, dtype, fill=1.0)
             self.k_norm = _param((dim,), device, dtype, fill=1.0)
+        self.wide_norm = bool(wide_norm)
+        if wide_norm:
+            self.q_norm = _param((self.nq,), device, dtype, fill=1.0)
+            self.k_norm = _param((self.nk,), device, dtype, fill=1.0)
+        self.q_scale = None
+        if q_temp:
+            # floor((p + 1) / every) in float64: exact where it is a whole number
+            n = torch.floor((torch.arange(max_pos, dtype=torch.float64) + 1.0) / float(q_temp["every"]))
+            self.q_scale = (1.0 + float(q_temp["coef"]) * torch.log(n + 1.0)).float().to(device)
         if slopes not in (None, "pow2"):
             raise ValueError(f"unknown distance slopes {slopes!r}")
         self.slopes = None
@@ -394,8 +424,14 @@ class GroupedAttention(torch.nn.Module):
         self.lam = float(self.vmix.data.float().item())
         if self.norm_weight:
             self.qk_w32 = torch.stack([self.q_norm.data.float(), self.k_norm.data.float()]).contiguous()
+        if self.wide_norm:
+            self.qk_w32 = torch.cat([self.q_norm.data.float(), self.k_norm.data.float()])
         if hasattr(self, "sink"):
             self.sink_logits = self.sink.data.float()
+
+    @property
+    def owns_cache(self) -> bool:
+        return self._src is None
 
     def kv_spec(self):
         return 1, self.Hkv, self.dim + self.vdim  # (planes, heads, row): [key | value] per kv head
@@ -418,39 +454,52 @@ class GroupedAttention(torch.nn.Module):
                 raise ValueError("value mixing needs the same kv heads x value size in all layers that use it")
             if v_first is None:
                 v_first = shared["v_first"] = torch.empty(T, self.nv, dtype=torch.float32, device=h.device)
-        sm.qkv_rope_cache(p, self.bias32, meta.positions, self.cos_sin, self.Hq, self.Hkv, self.dim, self.vdim,
-                          self.rot_dims, self.interleaved, self.eps if self.unit_norm else None, v_first, mode,
-                          self.lam, meta.slot_mapping, self.cache, q, self.qk_w32, self.norm_first, self.v_from_k,
-                          self.conv.weight if self.conv else None, self.conv.state if self.conv else None, meta.seq)
+        own = self._src is None
+        sm.qkv_rope_cache(p, self.bias32, meta.positions, self.cos_sin, self.Hq, self.Hkv if own else 0, self.dim,
+                          self.vdim, self.rot_dims, self.interleaved, self.eps if self.unit_norm or self.wide_norm else None,
+                          v_first, mode, self.lam, meta.slot_mapping, self.cache if own else None, q, self.qk_w32,
+                          self.norm_first, self.v_from_k, self.conv.weight if self.conv else None,
+                          self.conv.state if self.conv else None, meta.seq, self.wide_norm, self.q_scale)
         n0 = self.nq + self.nk + self.nv
         gate = p[:, n0:n0 + self.Hq * self.vdim] if self.has_gate else None
-        o = sm.grouped_attention(q, self.cache, self.dim, self.vdim, self.scale, meta.seq, gate, self.slopes,
+        o = sm.grouped_attention(q, self.cache if own else self._src[0].cache, self.dim, self.vdim, self.scale, meta.seq, gate, self.slopes,
                                  self.chunk, self.sink_logits, self.win, self.keep_first)
         return self.o(o)
 
 
 class GatedMLP(torch.nn.Module):
-    """W_down (act(W_gate h) * (W_up h)), gate and up as one projection; act "gelu_tanh" or "silu"."""
+    """W_down (act(W_gate h) * (W_up h)), gate and up as one projection; act "gelu_tanh" or "silu". act
+    "swish_limit": g sigmoid(1.702 g) (u + 1) with g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit)."""
 
-    def __init__(self, d_model, ff, act, device, dtype):
+    def __init__(self, d_model, ff, act, device, dtype, limit=0.0):
         super().__init__()
-        self.ff, self.act = ff, act
+        self.ff, self.act, self.limit = ff, act, float(limit)
         self.gate_up = ColumnLinear(d_model, 2 * ff, shard=False, device=device, dtype=dtype)
         self.down = ColumnLinear(ff, d_model, shard=False, device=device, dtype=dtype)
 
     def forward(self, h):
-        return self.down(sm.gated_act(self.gate_up(h), self.ff, self.act))
+        return self.down(sm.gated_act(self.gate_up(h), self.ff, self.act, self.limit))
 
 
 class ScoreMoE(torch.nn.Module):
     """Gated experts chosen by score: router outputs over ``experts + identity`` entries in fp32,
     scores = softmax over all of them, the ``top`` largest of score + correction chosen, weights = the
-    chosen scores over their sum. The last ``identity`` entries have no weights: they return their
-    input."""
+    chosen scores over their sum, times ``scale``. The last ``identity`` entries have no weights: they
+    return their input.
 
-    def __init__(self, d_model, ff, experts, identity, top, act, device, dtype):
+    groups, keep  the entries form ``groups`` equal groups of neighbours; only those of the ``keep`` groups whose
+                  largest score + correction is largest can be chosen
+    limit         of the "swish_limit" units (``GatedMLP``)
+    shared        a feed-forward that runs for every token and is added"""
+
+    def __init__(self, d_model, ff, experts, identity, top, act, device, dtype, limit=0.0, groups=1, keep=1, scale=1.0,
+                 shared=None):
         super().__init__()
+        if (experts + identity) % groups or not 1 <= keep <= groups or top > (experts + identity) // groups * keep:
+            raise ValueError(f"{top} of {experts + identity} entries in {groups} groups, {keep} of them kept")
         self.E, self.I, self.k, self.act = experts, identity, top, act
+        self.limit, self.groups, self.keep, self.scale = float(limit), int(groups), int(keep), float(scale)
+        self.shared = shared
         self.router = _param((experts + identity, d_model), device, dtype)
         self.correction = _param((experts + identity,), device, dtype, fill=0.0)
         self.w1 = _param((experts, 2 * ff, d_model), device, dtype)   # [gate rows | up rows]
@@ -463,8 +512,9 @@ class ScoreMoE(torch.nn.Module):
 
     def forward(self, h):
         logits = F.linear(h.float(), self.router32)
-        ids, w = sm.moe_route_scores(logits, self.correction32, self.k)
-        return sm.moe_gated_ffn(h, ids, w, self.w1, self.w2, self.act)
+        ids, w = sm.moe_route_scores(logits, self.correction32, self.k, self.groups, self.keep, self.scale)
+        return sm.moe_gated_ffn(h, ids, w, self.w1, self.w2, self.act, limit=self.limit,
+                                extra=self.shared(h) if self.shared is not None else None)
 
 
 class GatedDeltaMixer(torch.nn.Module):
@@ -760,3 +810,45 @@ class ResidualGates(torch.nn.Module):
 
     def forward(self, h):
         return self.proj(h)
+
+
+class RetentionMixer(torch.nn.Module):
+    """Linear attention whose state forgets with a fixed decay per head. One projection of the layer input gives
+    [q | k | v | g]: q and k (heads x ``dim``) are rotated (``rot`` {dims, base}, half-split pairs, or None), k is
+    multiplied by dim^-1/2. Per head, in fp32:
+
+        S <- decay S + k v^T;  o = S^T q
+
+    then o divided by its root mean square, times silu(g) unless ``gate`` is off, and the output projection.
+    State per sequence: S [heads, dim, vdim] fp32."""
+
+    def __init__(self, d_model, heads, dim, vdim, decay, rot, eps, max_pos, device, dtype, gate=True):
+        super().__init__()
+        if len(decay) != heads:
+            raise ValueError(f"{heads} heads and {len(decay)} decays")
+        self.H, self.dk, self.dv, self.eps, self.has_gate = heads, dim, vdim, eps, bool(gate)
+        self.nq, self.nv = heads * dim, heads * vdim
+        n = 2 * self.nq + self.nv * (2 if gate else 1)
+        self.proj = ColumnLinear(d_model, -(-n // 8) * 8, shard=False, device=device, dtype=dtype)
+        self.o = ColumnLinear(self.nv, d_model, shard=False, device=device, dtype=dtype)
+        self.rot_dims, self.cos_sin = 0, None
+        if rot:
+            self.rot_dims = int(rot["dims"])
+            if self.rot_dims > dim or self.rot_dims % 2:
+                raise ValueError(f"rotary dims {self.rot_dims} do not fit the head size {dim}")
+            self.cos_sin = rope_table(self.rot_dims, rot["base"], max_pos, device, rot.get("scaling"))
+        # decay^n, n = 0 .. a chunk's length, taken in float64
+        n = torch.arange(sm.RETENTION_CHUNK + 1, dtype=torch.float64)
+        self.powers = (torch.tensor(decay, dtype=torch.float64)[:, None] ** n).float().to(device)
+        self.state = None
+
+    def state_shapes(self):
+        return [((self.H, self.dk, self.dv), torch.float32)]
+
+    def bind_state(self, tensors):
+        (self.state,) = tensors
+
+    def forward(self, h, meta: AttnMeta):
+        y = sm.retention(self.proj(h), self.H, self.dk, self.dv, self.has_gate, meta.positions, self.cos_sin,
+                         self.rot_dims, self.powers, self.eps, self.state, meta.seq)
+        return self.o(y)

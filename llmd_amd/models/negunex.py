@@ -26,9 +26,9 @@ import torch
 
 from llmd_amd.engine.attn_meta import AttnMeta
 from llmd_amd.engine.config import ModelConfig
-from llmd_amd.ops import seqmix as sm
 from llmd_amd.parallel.state import get_state
 
+from .hyper import HyperConnection, stream_stack
 from .layers import LMHead, VocabEmbedding
 from .mixers import GatedMLP, GroupedAttention, ScoreMoE, _param
 
@@ -51,22 +51,6 @@ def make_mlp(m, d: int, device, dtype):
         r = m["router"]
         return ScoreMoE(d, m["expert"]["ff"], r["experts"], r.get("identity", 0), r["top"], "silu", device, dtype)
     raise ValueError(f"unknown feed-forward kind {m['kind']!r}")
-
-
-class HyperConnection(torch.nn.Module):
-    """The three tensors of one sublayer's connection to the streams; fp32 copies for the kernels."""
-
-    def __init__(self, S: int, learned: bool, device, dtype):
-        super().__init__()
-        self.learned = learned
-        self.w_in = _param((S,), device, dtype, fill=1.0)
-        self.w_out = _param((S,), device, dtype, fill=1.0)
-        self.mix = torch.nn.Parameter(torch.eye(S, device=device, dtype=dtype), requires_grad=False)
-        self.in32 = self.out32 = self.mix32 = None
-
-    def finalize(self):
-        self.in32, self.out32 = self.w_in.data.float(), self.w_out.data.float()
-        self.mix32 = self.mix.data.float().contiguous()
 
 
 class NegunexLayer(torch.nn.Module):
@@ -115,38 +99,16 @@ class NegunexForCausalLM(torch.nn.Module):
     def kv_specs(self):
         return [a.kv_spec() for a in self.attention_layers()]
 
-    def _sublayers(self):
-        """(connection, norm weight, callable) of every sublayer in order."""
-        out = []
-        for l in self.layers:
-            out.append((l.hc1, l.norm1, l.mix, True, False))
-            if l.mlp is not None:
-                out.append((l.hc2, l.norm2, l.mlp, False, True))
-            out[-1] = out[-1][:4] + (True,)
-        return out
-
     @torch.no_grad()
     def forward(self, input_ids, meta: AttnMeta, layer_out=None):
         """``layer_out``: optional list that receives the sum of the streams after every layer."""
-        T = input_ids.shape[0]
-        d, eps, dt = self.cfg.hidden_size, self.cfg.rms_norm_eps, self.dtype
-        X = torch.empty(self.S, T, d, dtype=torch.float32, device=input_ids.device)
-        sm.hyper_embed(input_ids, self.embed.weight, X)
-        subs = self._sublayers()
-        shared = {}
-        h = sm.hyper_norm(X, subs[0][0].in32, subs[0][1], eps, dt) if subs else None
-        for i, (hc, _, fn, is_mixer, ends_layer) in enumerate(subs):
-            y = fn(h, meta, shared) if is_mixer else fn(h)
-            if i + 1 < len(subs):
-                nxt_in, nxt_w = subs[i + 1][0].in32, subs[i + 1][1]
-            else:
-                nxt_in, nxt_w = self.ones, self.norm
-            h = sm.hyper_update_norm(X, y, hc.mix32, hc.out32, nxt_in, nxt_w, eps, dt)
-            if ends_layer and layer_out is not None:
-                layer_out.append(X.sum(0))
-        if not subs:
-            h = sm.hyper_norm(X, self.ones, self.norm, eps, dt)
-        return h
+        shared, subs = {}, []
+        for l in self.layers:
+            subs.append((l.hc1, l.norm1, lambda h, m=l.mix: m(h, meta, shared), l.mlp is None))
+            if l.mlp is not None:
+                subs.append((l.hc2, l.norm2, l.mlp, True))
+        return stream_stack(input_ids, self.embed.weight, self.ones, subs, self.norm, self.cfg.rms_norm_eps, self.dtype,
+                            layer_out=layer_out)
 
     @torch.no_grad()
     def compute_logits(self, h):

@@ -9,7 +9,8 @@ with the first norm, plain RMS norms of projections, the input convolution, the 
 HGRN2 recurrence, sliding windows with kept first tokens, keys as values, per-head gates of latent
 attention; two input convolutions over one state, the short convolution of q, k and v in the rotary /
 cache kernel, windows in latent attention, PolyNorm, the gated residual add, squared-ReLU experts beside
-a gated shared expert.
+a gated shared expert; RMS norms over hyper-connected streams, norms over whole projections and queries
+scaled by position in the rotary / cache kernel, clamped gated units, routing inside the best groups, retention.
 
 GPU tensors go to the ``llmd_amd._C_seqmix`` library (csrc/seqmix/*.hip, built on its own so a
 model that needs only these kernels compiles only these); it is templated on the activation
@@ -223,8 +224,8 @@ def moe_ffn(h, ids, w, w1, w2, act: str = "gelu", extra=None, extra_gate=None):
     C.moe_group(ids, E, slot_row, tile_e, pair_slot)
     a = torch.empty(max_tiles * MOE_TILE, Fh, dtype=h.dtype, device=dev)
     y = torch.empty(max_tiles * MOE_TILE, d, dtype=h.dtype, device=dev)
-    C.moe_gemm(h, k, slot_row, tile_e, w1, a, UNGATED_ACTS[act], n, None)   # n = rows of the step: picks the tile width
-    C.moe_gemm(a, 0, slot_row, tile_e, w2, y, 0, n, None)
+    C.moe_gemm(h, k, slot_row, tile_e, w1, a, UNGATED_ACTS[act], n, None, 0.0)   # n = rows of the step: picks the tile width
+    C.moe_gemm(a, 0, slot_row, tile_e, w2, y, 0, n, None, 0.0)
     out = torch.empty_like(h)
     C.moe_combine(y, pair_slot, w, out, None, extra, extra_gate)
     return out
@@ -238,30 +239,31 @@ def hyper_embed(ids, table, X):
     native().hyper_embed(ids, table, X)
 
 
-def hyper_norm(X, w_in, norm_w, eps: float, out_dtype):
-    """Layer norm (weight, no bias; two-pass fp32 variance) of u = sum_s w_in[s] X[s]."""
+def hyper_norm(X, w_in, norm_w, eps: float, out_dtype, rms: bool = False):
+    """Layer norm (weight, no bias; two-pass fp32 variance) of u = sum_s w_in[s] X[s]; ``rms``: its RMS norm."""
     if not X.is_cuda:
-        return ref.hyper_norm(X, w_in, norm_w, eps, out_dtype)
+        return ref.hyper_norm(X, w_in, norm_w, eps, out_dtype, rms)
     out = torch.empty(X.shape[1:], dtype=out_dtype, device=X.device)
-    native().hyper_norm(X, w_in, norm_w, float(eps), out)
+    native().hyper_norm(X, w_in, norm_w, float(eps), out, bool(rms))
     return out
 
 
-def hyper_update_norm(X, y, mix, w_out, next_in=None, next_w=None, eps: float = 0.0, out_dtype=None):
+def hyper_update_norm(X, y, mix, w_out, next_in=None, next_w=None, eps: float = 0.0, out_dtype=None,
+                      rms: bool = False):
     """X[t] <- sum_s mix[s, t] X[s] + w_out[t] y for all streams at once, in place (fp32); with
-    ``next_w`` also returns the layer norm of sum_s next_in[s] X[s], the next sublayer's input (or
+    ``next_w`` also returns the layer norm (``rms``: the RMS norm) of sum_s next_in[s] X[s], the next sublayer's input (or
     the model's final norm over the plain sum), from the same pass."""
     if not X.is_cuda:
-        return ref.hyper_update_norm(X, y, mix, w_out, next_in, next_w, eps, out_dtype)
+        return ref.hyper_update_norm(X, y, mix, w_out, next_in, next_w, eps, out_dtype, rms)
     out = torch.empty(X.shape[1:], dtype=out_dtype, device=X.device) if next_w is not None else None
-    native().hyper_update_norm(X, y, mix, w_out, next_in, next_w, float(eps), out)
+    native().hyper_update_norm(X, y, mix, w_out, next_in, next_w, float(eps), out, bool(rms))
     return out
 
 
 # ---- grouped-query attention with its own key and value sizes
 def qkv_rope_cache(qkv, bias, positions, cos_sin, Hq, Hkv, dim, vdim, rot_dims, interleaved, unit_eps, v_first,
                    v_mode, lam, slots, cache, q_out, qk_w=None, norm_first: bool = False, v_from_k: bool = False,
-                   conv_w=None, conv_state=None, seq=None):
+                   conv_w=None, conv_state=None, seq=None, wide_norm: bool = False, q_scale=None):
     """From a fused projection [q | k | v | ...] of a step's tokens: add ``bias`` (fp32, over q|k|v),
     rotate the first ``rot_dims`` dimensions of every query and key head by the angles of ``cos_sin``
     [max_pos, rot_dims] = [cos | sin] (pairs (2i, 2i+1) when ``interleaved``, (i, i + rot_dims/2)
@@ -278,16 +280,20 @@ def qkv_rope_cache(qkv, bias, positions, cos_sin, Hq, Hkv, dim, vdim, rot_dims, 
     causal convolution over time, y_t = sum_j w[:, j] u_(t - taps + 1 + j) with zeros before position 0; a
     token's earlier values come from the step's rows or from ``conv_state`` [slots, taps - 1, columns]
     (the sequence's last projected rows, without the bias), which is rolled forward to the run's end;
-    ``seq`` describes the step."""
+    ``seq`` describes the step.
+    ``wide_norm``: instead of every head, ALL q columns and all k columns of a token are divided by their root
+    mean square (``unit_eps``) and multiplied by ``qk_w`` fp32 [q columns + k columns], before the rotation.
+    ``q_scale`` fp32 [max_pos]: the query at position p is multiplied by q_scale[p].
+    ``Hkv`` 0: the projection has queries only; nothing is cached (``cache`` None)."""
     if not qkv.is_cuda:
         return ref.qkv_rope_cache(qkv, bias, positions, cos_sin, Hq, Hkv, dim, vdim, rot_dims, interleaved, unit_eps,
                                   v_first, v_mode, lam, slots, cache, q_out, qk_w, norm_first, v_from_k,
-                                  conv_w, conv_state, seq)
+                                  conv_w, conv_state, seq, wide_norm, q_scale)
     cv = (conv_w, conv_state, seq.row_seq, seq.seq_start, seq.seq_slot, seq.seq_init, int(seq.max_q)) \
         if conv_w is not None else (None,) * 6 + (0,)
     native().qkv_rope_cache(qkv, bias, positions, cos_sin, Hq, Hkv, dim, vdim, rot_dims, bool(interleaved),
                             unit_eps is not None, float(unit_eps or 0.0), v_first, int(v_mode), float(lam), slots, cache,
-                            q_out, qk_w, bool(norm_first), bool(v_from_k), *cv)
+                            q_out, qk_w, bool(norm_first), bool(v_from_k), *cv, bool(wide_norm), q_scale)
 
 
 GQA_MFMA = os.environ.get("LLMD_GQA_MFMA", "1") == "1"
@@ -357,31 +363,37 @@ def grouped_attention(q, cache, dim, vdim, scale: float, seq, gate=None, slopes=
     return out
 
 
-ACT_KINDS = {"gelu_tanh": 0, "silu": 1}
+ACT_KINDS = {"gelu_tanh": 0, "silu": 1, "swish_limit": 2}
 
 
-def gated_act(gu, Fh: int, kind: str):
-    """act(gu[:, :Fh]) * gu[:, Fh:], act the tanh form of GELU or SiLU, fp32 arithmetic."""
+def gated_act(gu, Fh: int, kind: str, limit: float = 0.0):
+    """act(gu[:, :Fh]) * gu[:, Fh:], act the tanh form of GELU or SiLU, fp32 arithmetic. "swish_limit":
+    g sigmoid(1.702 g) (u + 1) with g = min(gu[:, :Fh], limit) and u = clamp(gu[:, Fh:], -limit, limit)."""
     if not gu.is_cuda:
-        return ref.gated_act(gu, Fh, kind)
+        return ref.gated_act(gu, Fh, kind, limit)
     out = torch.empty(gu.shape[0], Fh, dtype=gu.dtype, device=gu.device)
-    native().gated_act(gu, int(Fh), ACT_KINDS[kind], out)
+    native().gated_act(gu, int(Fh), ACT_KINDS[kind], out, float(limit))
     return out
 
 
-def moe_route_scores(logits, correction, k: int):
+def moe_route_scores(logits, correction, k: int, groups: int = 1, keep: int = 1, scale: float = 1.0):
     """Scores = softmax over ALL router outputs (fp32); the k largest of score + correction are
-    chosen (ties: lower index); weights = the chosen scores / (their sum + 1e-20)."""
+    chosen (ties: lower index); weights = the chosen scores / (their sum + 1e-20) * scale. ``groups`` > 1: the
+    outputs form that many equal groups of neighbours, and only those of the ``keep`` groups whose largest
+    score + correction is largest (ties: lower index) can be chosen."""
     if not logits.is_cuda:
-        return ref.moe_route_scores(logits, correction, k)
+        return ref.moe_route_scores(logits, correction, k, groups, keep, scale)
     T = logits.shape[0]
     ids = torch.empty(T, k, dtype=torch.int32, device=logits.device)
     w = torch.empty(T, k, dtype=torch.float32, device=logits.device)
-    native().moe_route_scores(logits, correction, k, ids, w)
+    native().moe_route_scores(logits, correction, k, ids, w, int(groups), int(keep), float(scale))
     return ids, w
 
 
-def moe_gated_ffn(h, ids, w, w1, w2, kind: str = "silu", scale_input: bool = False):
+GATED_ACTS = {"gelu_tanh": 2, "silu": 3, "swish_limit": 5}
+
+
+def moe_gated_ffn(h, ids, w, w1, w2, kind: str = "silu", scale_input: bool = False, limit: float = 0.0, extra=None):
     """sum_j w[t, j] * W2[e] (act(Wg[e] h_t) * (Wu[e] h_t)), e = ids[t, j]; w1 [E, 2F, d] holds
     [gate rows | up rows], w2 [E, d, F]. ids >= E name identity experts: their output is h_t itself.
     Same grouping, tile GEMMs and fp32 combine as ``moe_ffn``; the activation and the product are the
@@ -390,9 +402,10 @@ def moe_gated_ffn(h, ids, w, w1, w2, kind: str = "silu", scale_input: bool = Fal
     ``scale_input``: the weight multiplies the expert's input instead of its output,
     sum_j W2[e] (act(Wg[e] (w h_t)) * (Wu[e] (w h_t))): the first GEMM's fp32 sums are scaled by the
     pair's weight before the activation (both products are linear in the input) and the combine adds
-    the rows as they are. No identity experts in this form."""
+    the rows as they are. No identity experts in this form.
+    ``limit``: of the "swish_limit" units (``gated_act``). ``extra`` [T, d]: a shared expert's result, added."""
     if not h.is_cuda:
-        return ref.moe_gated_ffn(h, ids, w, w1, w2, kind, scale_input)
+        return ref.moe_gated_ffn(h, ids, w, w1, w2, kind, scale_input, limit, extra)
     C = native()
     T, d = h.shape
     k = ids.shape[1]
@@ -407,10 +420,10 @@ def moe_gated_ffn(h, ids, w, w1, w2, kind: str = "silu", scale_input: bool = Fal
     C.moe_group(ids, E, slot_row, tile_e, pair_slot)
     a = torch.empty(max_tiles * MOE_TILE, Fh, dtype=h.dtype, device=dev)
     y = torch.empty(max_tiles * MOE_TILE, d, dtype=h.dtype, device=dev)
-    C.moe_gemm(h, k, slot_row, tile_e, w1, a, 2 + ACT_KINDS[kind], n, w if scale_input else None)
-    C.moe_gemm(a, 0, slot_row, tile_e, w2, y, 0, n, None)
+    C.moe_gemm(h, k, slot_row, tile_e, w1, a, GATED_ACTS[kind], n, w if scale_input else None, float(limit))
+    C.moe_gemm(a, 0, slot_row, tile_e, w2, y, 0, n, None, 0.0)
     out = torch.empty_like(h)
-    C.moe_combine(y, pair_slot, None if scale_input else w, out, h, None, None)
+    C.moe_combine(y, pair_slot, None if scale_input else w, out, h, extra, None)
     return out
 
 
@@ -572,4 +585,34 @@ def poly_norm(z, coef, eps: float):
         return ref.poly_norm(z, coef, eps)
     out = torch.empty(z.shape, dtype=z.dtype, device=z.device)
     native().poly_norm(z, *(float(v) for v in coef), float(eps), out)
+    return out
+
+
+# ---- retention
+RETENTION_CHUNK = 64  # tokens per chunk of the matrix form (csrc/seqmix/sm_retention.hip)
+
+
+def retention(p, H: int, dk: int, dv: int, gate: bool, positions, cos_sin, rot_dims: int, powers, eps: float, state, seq):
+    """Retention over a step's runs. ``p`` [T, >= 2 H dk + H dv (+ H dv)] = [q | k | v (| g)] as projected. q and k
+    are rotated on their first ``rot_dims`` dimensions (half-split pairs, angles of ``cos_sin``; 0: not), k times
+    dk^-1/2; per head, all fp32, S <- decay S + k v^T; o = S^T q; the result is o / rms(o) (times silu(g) with
+    ``gate``). ``powers`` fp32 [H, RETENTION_CHUNK + 1] = decay^n. ``state`` [slots, H, dk, dv] fp32 is
+    continued (seq_init) and written back. Returns [T, H dv].
+
+    Sequences that bring one token advance their state in one pass. Longer runs take the chunked matrix form: in a
+    chunk of n tokens that starts from S, o_i = decay^(i+1) S^T q_i + sum_{j<=i} decay^(i-j) (q_i . k_j) v_j
+    and the state it leaves is decay^n S + sum_j decay^(n-1-j) k_j v_j^T."""
+    out = torch.empty(p.shape[0], H * dv, dtype=p.dtype, device=p.device)
+    if not p.is_cuda:
+        return ref.retention(p, H, dk, dv, gate, positions, cos_sin, rot_dims, powers, eps, state, seq.seq_start,
+                             seq.seq_slot, seq.seq_init, out)
+    # the step's single tokens come first; what follows them is cut into chunks
+    nd = 0
+    for n in seq.q_lens:
+        if n != 1:
+            break
+        nd += 1
+    chunks, nc = (None, 0) if nd == len(seq.q_lens) else seq.scan_chunks(RETENTION_CHUNK)
+    native().retention(p, int(H), int(dk), int(dv), bool(gate), positions, cos_sin, int(rot_dims), powers, float(eps),
+                       state, seq.seq_start, seq.seq_slot, seq.seq_init, out, nd, chunks, nc)
     return out

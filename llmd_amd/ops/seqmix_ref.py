@@ -182,19 +182,20 @@ def hyper_embed(ids, table, X):
     X.copy_(table[ids].float().unsqueeze(0).expand_as(X))
 
 
-def hyper_norm(X, w_in, norm_w, eps, out_dtype):
-    return _ln((X * w_in.view(-1, 1, 1)).sum(0), norm_w, eps).to(out_dtype)
+def hyper_norm(X, w_in, norm_w, eps, out_dtype, rms=False):
+    u = (X * w_in.view(-1, 1, 1)).sum(0)
+    return (_rms(u, eps) * norm_w.float() if rms else _ln(u, norm_w, eps)).to(out_dtype)
 
 
-def hyper_update_norm(X, y, mix, w_out, next_in, next_w, eps, out_dtype):
+def hyper_update_norm(X, y, mix, w_out, next_in, next_w, eps, out_dtype, rms=False):
     new = torch.einsum("st,snd->tnd", mix, X) + w_out.view(-1, 1, 1) * y.float().unsqueeze(0)
     X.copy_(new)
-    return None if next_w is None else hyper_norm(X, next_in, next_w, eps, out_dtype)
+    return None if next_w is None else hyper_norm(X, next_in, next_w, eps, out_dtype, rms)
 
 
 def qkv_rope_cache(qkv, bias, positions, cos_sin, Hq, Hkv, dim, vdim, rot_dims, interleaved, unit_eps, v_first,
                    v_mode, lam, slots, cache, q_out, qk_w=None, norm_first=False, v_from_k=False, conv_w=None,
-                   conv_state=None, seq=None):
+                   conv_state=None, seq=None, wide_norm=False, q_scale=None):
     T = qkv.shape[0]
     nq, nk, nv = Hq * dim, Hkv * dim, 0 if v_from_k else Hkv * vdim
     x = qkv[:, :nq + nk + nv].float()
@@ -202,6 +203,10 @@ def qkv_rope_cache(qkv, bias, positions, cos_sin, Hq, Hkv, dim, vdim, rot_dims, 
         x = x + bias.float()
     if conv_w is not None:
         x = _conv_columns(x, qkv[:, :nq + nk + nv], bias, positions, conv_w, conv_state, seq)
+    if wide_norm:
+        x = torch.cat([_rms(x[:, :nq], unit_eps) * qk_w[:nq], _rms(x[:, nq:nq + nk], unit_eps) * qk_w[nq:], x[:, nq + nk:]],
+                      -1)
+        unit_eps = None
     q, k = x[:, :nq].view(T, Hq, dim), x[:, nq:nq + nk].view(T, Hkv, dim)
     v = k if v_from_k else x[:, nq + nk:].view(T, Hkv, vdim)
 
@@ -235,7 +240,11 @@ def qkv_rope_cache(qkv, bias, positions, cos_sin, Hq, Hkv, dim, vdim, rot_dims, 
         v_first.copy_(v.reshape(T, nv))
     elif v_mode == 2:
         v = (1.0 - lam) * v + lam * v_first.view(T, Hkv, vdim)
+    if q_scale is not None:
+        q = q * q_scale[positions].view(T, 1, 1)
     q_out.copy_(q.to(q_out.dtype))
+    if Hkv == 0:
+        return
     nb, _, bs, _ = cache.shape
     kc, vc = kv_views(cache, dim, vdim)
     ok = slots >= 0
@@ -302,22 +311,31 @@ def grouped_attention(q, cache, dim, vdim, tables, row_seq, row_len, scale, gate
     return out
 
 
-def _act(z, kind):
-    return F.gelu(z, approximate="tanh") if kind == "gelu_tanh" else F.silu(z)
+def _gated(g, u, kind, limit=0.0):
+    if kind == "swish_limit":
+        g, u = g.clamp(max=limit), u.clamp(-limit, limit)
+        return g * torch.sigmoid(1.702 * g) * (u + 1.0)
+    return (F.gelu(g, approximate="tanh") if kind == "gelu_tanh" else F.silu(g)) * u
 
 
-def gated_act(gu, Fh, kind):
-    return (_act(gu[:, :Fh].float(), kind) * gu[:, Fh:2 * Fh].float()).to(gu.dtype)
+def gated_act(gu, Fh, kind, limit=0.0):
+    return _gated(gu[:, :Fh].float(), gu[:, Fh:2 * Fh].float(), kind, limit).to(gu.dtype)
 
 
-def moe_route_scores(logits, correction, k):
+def moe_route_scores(logits, correction, k, groups=1, keep=1, scale=1.0):
     s = torch.softmax(logits.float(), -1)
-    ids = (s + correction.float()).topk(k, -1).indices
+    c = s + correction.float()
+    if groups > 1:
+        T, n = c.shape
+        best = c.view(T, groups, n // groups).max(-1).values.sort(dim=-1, descending=True, stable=True).indices[:, :keep]
+        kept = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, best, True)
+        c = c.masked_fill(~kept.repeat_interleave(n // groups, 1), -math.inf)
+    ids = c.topk(k, -1).indices
     w = torch.gather(s, 1, ids)
-    return ids.int(), w / (w.sum(-1, keepdim=True) + 1e-20)
+    return ids.int(), w / (w.sum(-1, keepdim=True) + 1e-20) * scale
 
 
-def moe_gated_ffn(h, ids, w, w1, w2, kind, scale_input=False):
+def moe_gated_ffn(h, ids, w, w1, w2, kind, scale_input=False, limit=0.0, extra=None):
     """w1 [E, 2F, d] = [gate | up] rows, w2 [E, d, F]; ids >= E are identity experts."""
     if scale_input:
         E, F2, _ = w1.shape
@@ -326,7 +344,7 @@ def moe_gated_ffn(h, ids, w, w1, w2, kind, scale_input=False):
         for e in ids.unique().tolist():
             t, j = (ids == e).nonzero(as_tuple=True)
             gu = (hf[t] @ w1[e].float().T) * w[t, j, None]
-            a = (_act(gu[:, :F2 // 2], kind) * gu[:, F2 // 2:]).to(h.dtype).float()
+            a = _gated(gu[:, :F2 // 2], gu[:, F2 // 2:], kind, limit).to(h.dtype).float()
             out.index_add_(0, t, (a @ w2[e].float().T).to(h.dtype).float())
         return out.to(h.dtype)
     E, F2, _ = w1.shape
@@ -338,8 +356,10 @@ def moe_gated_ffn(h, ids, w, w1, w2, kind, scale_input=False):
             out.index_add_(0, t, hf[t] * w[t, j, None])
             continue
         gu = (hf[t] @ w1[e].float().T)
-        a = (_act(gu[:, :F2 // 2], kind) * gu[:, F2 // 2:]).to(h.dtype).float()
+        a = _gated(gu[:, :F2 // 2], gu[:, F2 // 2:], kind, limit).to(h.dtype).float()
         out.index_add_(0, t, (a @ w2[e].float().T).to(h.dtype).float() * w[t, j, None])
+    if extra is not None:
+        out += extra.float()
     return out.to(h.dtype)
 
 
@@ -476,3 +496,28 @@ def poly_norm(z, coef, eps):
     a, b, c, e = coef
     v = z.float()
     return (a * _rms(v, eps) + b * _rms(v * v, eps) + c * _rms(v * v * v, eps) + e).to(z.dtype)
+
+
+# ---- retention
+def retention(p, H, dk, dv, gate, positions, cos_sin, rot_dims, powers, eps, state, seq_start, seq_slot, seq_init, out):
+    T, nq, nv = p.shape[0], H * dk, H * dv
+    q, k = p[:, :nq].float().view(T, H, dk), p[:, nq:2 * nq].float().view(T, H, dk)
+    if rot_dims:
+        cs = cos_sin[positions][:, None]
+        q, k = _rot(q, cs, rot_dims), _rot(k, cs, rot_dims)
+    k = k * dk ** -0.5
+    v = p[:, 2 * nq:2 * nq + nv].float().view(T, H, dv)
+    decay = powers[:, 1].view(H, 1, 1)
+    for i in range(seq_slot.numel()):
+        lo, hi, sl = int(seq_start[i]), int(seq_start[i + 1]), int(seq_slot[i])
+        if hi == lo:
+            continue
+        S = state[sl].clone() if int(seq_init[i]) else torch.zeros_like(state[sl])
+        for t in range(lo, hi):
+            S = decay * S + k[t][:, :, None] * v[t][:, None]
+            o = _rms((S * q[t][:, :, None]).sum(1), eps).reshape(nv)
+            if gate:
+                o = o * F.silu(p[t, 2 * nq + nv:2 * nq + 2 * nv].float())
+            out[t] = o.to(out.dtype)
+        state[sl] = S
+    return out
