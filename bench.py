@@ -95,13 +95,14 @@ def parse():
                         "(latent attention + experts, selective scan, delta rule beside DeepSeek-V2-Lite layers; "
                         "hyper-connected grouped attention beside Llama-3-8B and Qwen3-30B-A3B layers; Zumizen's gated "
                         "delta rules and chunked attention with input-scaled experts; Kakalorn's windowed attention, "
-                        "HGRN2 and latent attention with shared caches; Kokatar's parallel layers) at model-like "
+                        "HGRN2 and latent attention with shared caches; Kokatar's parallel layers; Koduzen's retention, "
+                        "position-free attention with shared keys and grouped routing) at model-like "
                         "sizes (llmd_amd/tools/mixer_bench.py; uses --isl as "
                         "the context and --concurrency as the decode batch when they are given)")
     p.add_argument("--mixer-only", default="",
                    help="with --mixer-bench: only the entries whose name starts with one of these (commas between), "
-                        "e.g. negunex,llama,qwen3, zumizen,delta,latent,negunex-moe, kakalorn,negunex-dense,llama or "
-                        "kokatar,kakalorn,llama")
+                        "e.g. negunex,llama,qwen3, zumizen,delta,latent,negunex-moe, kakalorn,negunex-dense,llama, "
+                        "kokatar,kakalorn,llama or koduzen,negunex,kakalorn-hgrn2,llama")
     p.add_argument("--steps", type=int, default=40)
     p.add_argument("--warmup", type=int, default=20)
     p.add_argument("--model", default="llama-3-70b")

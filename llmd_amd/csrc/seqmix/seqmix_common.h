@@ -54,8 +54,8 @@ template <typename T> struct Fn {
 };
 template <> struct Fn<uint16_t> {
   static __device__ __forceinline__ float exp(float x) { return __expf(x); }
-  static __device__ __forceinline__ float sigmoid(float x) { return __frcp_rn(1.f + __expf(-x)); }
-  static __device__ __forceinline__ float silu(float x) { return x * __frcp_rn(1.f + __expf(-x)); }
+  static __device__ __forceinline__ float sigmoid(float x) { return __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
+  static __device__ __forceinline__ float silu(float x) { return x * __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
   static __device__ __forceinline__ float softplus(float x) { return x > 20.f ? x : __logf(1.f + __expf(x)); }
   static __device__ __forceinline__ float rsqrt(float x) { return __frsqrt_rn(x); }
 };
@@ -63,10 +63,11 @@ template <> struct Fn<uint16_t> {
 __device__ __forceinline__ float siluf_(float x) { return x / (1.f + expf(-x)); }
 
 // Clamped gated unit: g sigmoid(1.702 g) (v + 1), g cut off above ``limit``, v on both sides.
+template <typename T>
 __device__ __forceinline__ float clamped_unit(float g, float v, float limit) {
   g = fminf(g, limit);
   v = fminf(fmaxf(v, -limit), limit);
-  return g / (1.f + expf(-1.702f * g)) * (v + 1.f);
+  return g * Fn<T>::sigmoid(1.702f * g) * (v + 1.f);
 }
 
 }  // namespace sm

@@ -36,7 +36,7 @@
 // token's earlier projections come from the step's own rows or from the sequence's state (its last
 // taps - 1 projected rows, stored without the bias), positions before 0 count as zeros; wide - all q columns and
 // all k columns of a token are divided by their own root mean square and weighted (qk_w: one weight per column)
-// before the rotation, every workgroup of the token forming both sums; q_scale [max_pos] - the query at position
+// before the rotation; q_scale [max_pos] - the query at position
 // p is multiplied by q_scale[p]; Hkv 0 - the projection has queries only and nothing is cached.
 #include "seqmix_common.h"
 #include <algorithm>
@@ -207,6 +207,84 @@ __device__ __forceinline__ void st8(bf16_t* p, const float (&v)[8], float mul) {
   *reinterpret_cast<uint4*>(p) = make_uint4(w[0], w[1], w[2], w[3]);
 }
 
+// The values of tg (1 or 8) tokens, a column per thread; ``unit`` numbers the workgroups of this part.
+template <int TAPS>
+__device__ __forceinline__ void value_part(int unit, const bf16_t* __restrict__ qkv, int64_t stride,
+                                           const float* __restrict__ bias, const int64_t* __restrict__ positions, int Hq,
+                                           int Hkv, int dim, int vdim, float* __restrict__ v_first, int v_mode, float lam,
+                                           const int64_t* __restrict__ slots, bf16_t* __restrict__ cache, int bs,
+                                           int v_from_k, const ConvArgs<bf16_t>& cv, int tg, int T) {
+  const int nv = Hkv * vdim, vcol0 = v_from_k ? Hq * dim : (Hq + Hkv) * dim, nvb = (nv + NT - 1) / NT;
+  const int e = (unit % nvb) * NT + threadIdx.x, t0 = unit / nvb * tg;
+  if (t0 >= T || e >= nv) return;
+  const int col = vcol0 + e, g = e / vdim, c = e - g * vdim;
+  const float vb = bias ? bias[col] : 0.f;
+  const int64_t vbase = (int64_t)g * bs * (dim + vdim) + (int64_t)bs * dim + (int64_t)c * bs;  // within a page
+  const int64_t page = (int64_t)Hkv * bs * (dim + vdim);
+  float w[TAPS > 0 ? TAPS : 1];
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) w[j] = ld(cv.w + (int64_t)col * TAPS + j);
+  const int64_t s0 = slots[t0];
+  const bool eight = tg == 8 && t0 + 8 <= T && s0 >= 0 && (s0 & 7) == 0 && (bs & 7) == 0 && slots[t0 + 7] == s0 + 7;
+  if (eight) {  // one page, hence one sequence
+    constexpr int PAST = TAPS > 1 ? TAPS - 1 : 0;
+    float u[8 + PAST];
+    if constexpr (PAST > 0) {
+      const int s = cv.row_seq[t0], run0 = t0 - cv.seq_start[s];
+      const int64_t pos0 = positions[t0];
+      const bf16_t* past = cv.state + (int64_t)cv.seq_slot[s] * PAST * cv.C;
+#pragma unroll
+      for (int k = 0; k < PAST; ++k) {
+        const int back = PAST - k;
+        u[k] = pos0 < back ? 0.f
+                           : ld(run0 >= back ? qkv + (t0 - back) * stride + col : past + (int64_t)(k + run0) * cv.C + col) + vb;
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) u[PAST + i] = ld(qkv + (t0 + i) * stride + col) + vb;
+    float v[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      if constexpr (TAPS > 0) {
+        v[i] = 0.f;
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) v[i] += w[j] * u[i + j];
+      } else {
+        v[i] = u[i];
+      }
+      if (v_mode == 1) v_first[(int64_t)(t0 + i) * nv + e] = v[i];
+      else if (v_mode == 2) v[i] = (1.f - lam) * v[i] + lam * v_first[(int64_t)(t0 + i) * nv + e];
+    }
+    st8(cache + s0 / bs * page + vbase + s0 % bs, v, 1.f);
+    return;
+  }
+  for (int t = t0; t < min(t0 + tg, T); ++t) {
+    const bf16_t* row = qkv + t * stride;
+    float v = ld(row + col) + vb;
+    if constexpr (TAPS > 0) v *= w[TAPS - 1];
+    if constexpr (TAPS > 1) {
+      const int s = cv.row_seq[t], run = t - cv.seq_start[s];
+      const int64_t pos = positions[t];
+      bf16_t* past = cv.state + (int64_t)cv.seq_slot[s] * (TAPS - 1) * cv.C;
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) {
+        const int back = TAPS - 1 - j;
+        if (pos >= back)
+          v += w[j] * (ld(run >= back ? row - back * stride + col : past + (int64_t)(j + run) * cv.C + col) + vb);
+      }
+      if (run == 0 && cv.seq_start[s + 1] == t + 1) {  // the run is this token
+#pragma unroll
+        for (int j = 0; j < TAPS - 2; ++j) past[(int64_t)j * cv.C + col] = past[(int64_t)(j + 1) * cv.C + col];
+        past[(int64_t)(TAPS - 2) * cv.C + col] = row[col];
+      }
+    }
+    if (v_mode == 1) v_first[(int64_t)t * nv + e] = v;
+    else if (v_mode == 2) v = (1.f - lam) * v + lam * v_first[(int64_t)t * nv + e];
+    const int64_t slot = slots[t];
+    if (slot >= 0) st(cache + slot / bs * page + vbase + slot % bs, v);
+  }
+}
+
 template <int TAPS>
 __global__ __launch_bounds__(NT) void qkv_rope_cache_vec_kernel(
     const bf16_t* __restrict__ qkv, int64_t stride, const float* __restrict__ bias,
@@ -214,78 +292,10 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_vec_kernel(
     int rot_dims, int interleaved, int unit, float eps, float* __restrict__ v_first, int v_mode, float lam,
     const int64_t* __restrict__ slots, bf16_t* __restrict__ cache, int bs, bf16_t* __restrict__ q_out,
     const float* __restrict__ qk_w, int norm_first, int v_from_k, ConvArgs<bf16_t> cv,
-    int gh, int tg, int T, int wide, const float* __restrict__ q_scale) {
+    int gh, int tg, int T, const float* __restrict__ q_scale) {
   if ((int)blockIdx.y >= gh) {
-    const int nv = Hkv * vdim, vcol0 = v_from_k ? Hq * dim : (Hq + Hkv) * dim, nvb = (nv + NT - 1) / NT;
-    const int unit = ((int)blockIdx.y - gh) * gridDim.x + blockIdx.x;
-    const int e = (unit % nvb) * NT + threadIdx.x, t0 = unit / nvb * tg;
-    if (t0 >= T || e >= nv) return;
-    const int col = vcol0 + e, g = e / vdim, c = e - g * vdim;
-    const float vb = bias ? bias[col] : 0.f;
-    const int64_t vbase = (int64_t)g * bs * (dim + vdim) + (int64_t)bs * dim + (int64_t)c * bs;  // within a page
-    const int64_t page = (int64_t)Hkv * bs * (dim + vdim);
-    float w[TAPS > 0 ? TAPS : 1];
-#pragma unroll
-    for (int j = 0; j < TAPS; ++j) w[j] = ld(cv.w + (int64_t)col * TAPS + j);
-    const int64_t s0 = slots[t0];
-    const bool eight = tg == 8 && t0 + 8 <= T && s0 >= 0 && (s0 & 7) == 0 && (bs & 7) == 0 && slots[t0 + 7] == s0 + 7;
-    if (eight) {  // one page, hence one sequence
-      constexpr int PAST = TAPS > 1 ? TAPS - 1 : 0;
-      float u[8 + PAST];
-      if constexpr (PAST > 0) {
-        const int s = cv.row_seq[t0], run0 = t0 - cv.seq_start[s];
-        const int64_t pos0 = positions[t0];
-        const bf16_t* past = cv.state + (int64_t)cv.seq_slot[s] * PAST * cv.C;
-#pragma unroll
-        for (int k = 0; k < PAST; ++k) {
-          const int back = PAST - k;
-          u[k] = pos0 < back ? 0.f
-                             : ld(run0 >= back ? qkv + (t0 - back) * stride + col : past + (int64_t)(k + run0) * cv.C + col) + vb;
-        }
-      }
-#pragma unroll
-      for (int i = 0; i < 8; ++i) u[PAST + i] = ld(qkv + (t0 + i) * stride + col) + vb;
-      float v[8];
-#pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        if constexpr (TAPS > 0) {
-          v[i] = 0.f;
-#pragma unroll
-          for (int j = 0; j < TAPS; ++j) v[i] += w[j] * u[i + j];
-        } else {
-          v[i] = u[i];
-        }
-        if (v_mode == 1) v_first[(int64_t)(t0 + i) * nv + e] = v[i];
-        else if (v_mode == 2) v[i] = (1.f - lam) * v[i] + lam * v_first[(int64_t)(t0 + i) * nv + e];
-      }
-      st8(cache + s0 / bs * page + vbase + s0 % bs, v, 1.f);
-      return;
-    }
-    for (int t = t0; t < min(t0 + tg, T); ++t) {
-      const bf16_t* row = qkv + t * stride;
-      float v = ld(row + col) + vb;
-      if constexpr (TAPS > 0) v *= w[TAPS - 1];
-      if constexpr (TAPS > 1) {
-        const int s = cv.row_seq[t], run = t - cv.seq_start[s];
-        const int64_t pos = positions[t];
-        bf16_t* past = cv.state + (int64_t)cv.seq_slot[s] * (TAPS - 1) * cv.C;
-#pragma unroll
-        for (int j = 0; j < TAPS - 1; ++j) {
-          const int back = TAPS - 1 - j;
-          if (pos >= back)
-            v += w[j] * (ld(run >= back ? row - back * stride + col : past + (int64_t)(j + run) * cv.C + col) + vb);
-        }
-        if (run == 0 && cv.seq_start[s + 1] == t + 1) {  // the run is this token
-#pragma unroll
-          for (int j = 0; j < TAPS - 2; ++j) past[(int64_t)j * cv.C + col] = past[(int64_t)(j + 1) * cv.C + col];
-          past[(int64_t)(TAPS - 2) * cv.C + col] = row[col];
-        }
-      }
-      if (v_mode == 1) v_first[(int64_t)t * nv + e] = v;
-      else if (v_mode == 2) v = (1.f - lam) * v + lam * v_first[(int64_t)t * nv + e];
-      const int64_t slot = slots[t];
-      if (slot >= 0) st(cache + slot / bs * page + vbase + slot % bs, v);
-    }
+    value_part<TAPS>(((int)blockIdx.y - gh) * gridDim.x + blockIdx.x, qkv, stride, bias, positions, Hq, Hkv, dim, vdim,
+                     v_first, v_mode, lam, slots, cache, bs, v_from_k, cv, tg, T);
     return;
   }
   const int64_t t = blockIdx.x;
@@ -307,31 +317,15 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_vec_kernel(
   const int64_t blk = slot >= 0 ? slot / bs : 0, off = slot >= 0 ? slot % bs : 0;
   const int lph = dim >> 3, hpp = NT / lph;  // lanes per head, heads per pass
   const int c = threadIdx.x & (lph - 1), hl = threadIdx.x / lph;
-  float inv_q = 1.f, inv_k = 1.f;  // wide: of the whole projections
-  if (wide) {
-    __shared__ float red[NT / 64];
-    float sq = 0.f, sk = 0.f;
-    for (int e = threadIdx.x * 8; e < (Hq + Hkv) * dim; e += NT * 8) {  // a head is whole pieces of eight
-      float v[8], s8 = 0.f;
-      ld8(row + e, v);
-      if (bias) add8(bias + e, v);
-#pragma unroll
-      for (int i = 0; i < 8; ++i) s8 += v[i] * v[i];
-      if (e < Hq * dim) sq += s8;
-      else sk += s8;
-    }
-    inv_q = 1.f / sqrtf(block_sum<NT>(sq, red) / (float)(Hq * dim) + eps);
-    if (Hkv > 0) inv_k = 1.f / sqrtf(block_sum<NT>(sk, red) / (float)(Hkv * dim) + eps);
-  }
-  if (q_scale) inv_q *= q_scale[pos];
+  const float q_mul = q_scale ? q_scale[pos] : 1.f;
   for (int h0 = blockIdx.y * hpp; h0 < Hq + Hkv; h0 += gh * hpp) {
     const int hd = h0 + hl;
     const bool on = hd < Hq + Hkv;
     const int col = hd * dim + c * 8;  // q heads, then k heads, back to back in the projection
     float x[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     float ss = 0.f;
-    const float* nw = qk_w ? qk_w + (wide ? hd * dim : hd < Hq ? 0 : dim) : nullptr;
-    const float* nw1 = (norm_first || wide) ? nw : nullptr;  // weights applied before the rotation
+    const float* nw = qk_w ? qk_w + (hd < Hq ? 0 : dim) : nullptr;
+    const float* nw1 = norm_first ? nw : nullptr;  // weights applied before the rotation
     if (on) {
       ld8(row + col, x);
       if (bias) add8(bias + col, x);
@@ -367,7 +361,7 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_vec_kernel(
               *reinterpret_cast<const uint4*>(row + col);
         }
       }
-      if (norm_first || wide) {
+      if (norm_first) {
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
           ss += x[i] * x[i];
@@ -414,7 +408,7 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_vec_kernel(
         }
       }
     }
-    float inv = hd < Hq ? inv_q : inv_k;
+    float inv = hd < Hq ? q_mul : 1.f;
     if (unit) {
       if (!norm_first) {
 #pragma unroll
@@ -430,6 +424,99 @@ __global__ __launch_bounds__(NT) void qkv_rope_cache_vec_kernel(
     }
     if (hd < Hq) st8(q_out + (t * Hq + hd) * dim + c * 8, x, inv);
     else if (slot >= 0) st8(cache + (blk * Hkv + (hd - Hq)) * bs * Dr + off * dim + c * 8, x, inv);
+  }
+}
+
+// Norms over whole projections, 16-byte form: one workgroup holds all q and k columns of a token in registers, eight
+// per thread and pass (NP passes of 2048 columns), forms both sums at once, and takes the rotation's partner values
+// from the lane that owns them (half-split pairs; a head is dim / 8 neighbouring lanes). Sizes as for the kernel above.
+template <int NP>
+__global__ __launch_bounds__(NT) void qkv_wide_cache_vec_kernel(
+    const bf16_t* __restrict__ qkv, int64_t stride, const float* __restrict__ bias,
+    const int64_t* __restrict__ positions, const float* __restrict__ cos_sin, int Hq, int Hkv, int dim, int vdim,
+    int rot_dims, float eps, float* __restrict__ v_first, int v_mode, float lam, const int64_t* __restrict__ slots,
+    bf16_t* __restrict__ cache, int bs, bf16_t* __restrict__ q_out, const float* __restrict__ qk_w,
+    ConvArgs<bf16_t> cv, int tg, int T, const float* __restrict__ q_scale) {
+  if (blockIdx.y > 0) {
+    value_part<0>(((int)blockIdx.y - 1) * gridDim.x + blockIdx.x, qkv, stride, bias, positions, Hq, Hkv, dim, vdim,
+                  v_first, v_mode, lam, slots, cache, bs, 0, cv, tg, T);
+    return;
+  }
+  __shared__ float red[2][NT / 64];
+  const int64_t t = blockIdx.x;
+  const bf16_t* row = qkv + t * stride;
+  const int nq = Hq * dim, nqk = (Hq + Hkv) * dim;
+  float x[NP][8];
+  float sq = 0.f, sk = 0.f;
+#pragma unroll
+  for (int i = 0; i < NP; ++i) {
+    const int col = (i * NT + threadIdx.x) * 8;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[i][j] = 0.f;
+    if (col < nqk) {
+      ld8(row + col, x[i]);
+      if (bias) add8(bias + col, x[i]);
+    }
+  }
+  const int64_t pos = positions[t], slot = slots[t];
+  const int half = rot_dims >> 1;
+  const float* cs = cos_sin + (rot_dims ? pos * rot_dims : 0);
+#pragma unroll
+  for (int i = 0; i < NP; ++i) {
+    float s8 = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) s8 += x[i][j] * x[i][j];
+    if ((i * NT + (int)threadIdx.x) * 8 < nq) sq += s8;
+    else sk += s8;
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if ((threadIdx.x & 63) == 0) {
+    red[0][threadIdx.x >> 6] = sq;
+    red[1][threadIdx.x >> 6] = sk;
+  }
+  __syncthreads();
+  sq = sk = 0.f;
+#pragma unroll
+  for (int i = 0; i < NT / 64; ++i) {
+    sq += red[0][i];
+    sk += red[1][i];
+  }
+  const float inv_q = 1.f / sqrtf(sq / (float)nq + eps) * (q_scale ? q_scale[pos] : 1.f);
+  const float inv_k = Hkv > 0 ? 1.f / sqrtf(sk / (float)(nqk - nq) + eps) : 0.f;
+  const int lph = dim >> 3, Dr = dim + vdim;
+  const int c = threadIdx.x & (lph - 1);  // the same in every pass: a pass is whole heads
+  const int64_t blk = slot >= 0 ? slot / bs : 0, off = slot >= 0 ? slot % bs : 0;
+  const bool turn = c * 8 < rot_dims, first = c * 8 < half;
+  const int src = turn ? (int)(threadIdx.x & 63) + (first ? half : -half) / 8 : (int)(threadIdx.x & 63);
+  float cc[8] = {1.f, 1.f, 1.f, 1.f, 1.f, 1.f, 1.f, 1.f}, sn[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+  if (turn) {
+#pragma unroll
+    for (int j = 0; j < 8; ++j) cc[j] = 0.f;
+    add8(cs + (first ? c * 8 : c * 8 - half), cc);
+    add8(cs + half + (first ? c * 8 : c * 8 - half), sn);
+  }
+#pragma unroll
+  for (int i = 0; i < NP; ++i) {
+    if (i * NT * 8 >= nqk) break;
+    const int col = (i * NT + threadIdx.x) * 8;
+    const bool on = col < nqk;
+    if (on) {
+      float w[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      add8(qk_w + col, w);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[i][j] *= w[j];
+    }
+    if (rot_dims > 0) {
+      float xp[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) xp[j] = __shfl(x[i][j], src, 64);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[i][j] = first ? x[i][j] * cc[j] - xp[j] * sn[j] : x[i][j] * cc[j] + xp[j] * sn[j];
+    }
+    if (!on) continue;
+    if (col < nq) st8(q_out + t * nq + col, x[i], inv_q);
+    else if (slot >= 0) st8(cache + (blk * Hkv + (col - nq) / dim) * bs * Dr + off * dim + c * 8, x[i], inv_k);
   }
 }
 
@@ -1226,18 +1313,32 @@ void sm_qkv_rope_cache(const void* qkv, int64_t stride, const float* bias, const
   else if (dim % 8 == 0 && dim <= 512 && ((dim >> 3) & ((dim >> 3) - 1)) == 0 && stride % 8 == 0 &&
            rot_dims % (interleaved ? 8 : 16) == 0 && taps <= 8 && (taps == 0 || (C % 8 == 0 && !v_from_k)) &&
            (((uintptr_t)qkv | (uintptr_t)q_out | (uintptr_t)cache | (uintptr_t)bias | (uintptr_t)cos_sin |
-             (uintptr_t)conv_w | (uintptr_t)conv_state) & 15) == 0) {
+             (uintptr_t)conv_w | (uintptr_t)conv_state) & 15) == 0 &&
+           (!wide || (!interleaved && (Hq + Hkv) * dim <= 8 * NT * 8 && ((uintptr_t)qk_w & 15) == 0))) {
     // a pass covers 256 / (dim / 8) heads: fewer workgroups per token than the element-wise form
     const int hpp = NT / (dim >> 3);
     const int per_tok_v = (Hq + Hkv + hpp - 1) / hpp;
     const int gh = std::max(1, std::min(per_tok_v, 4096 / T)), tg = T >= 256 ? 8 : 1;
     const int units = (T + tg - 1) / tg * ((Hkv * vdim + NT - 1) / NT);
-    const dim3 vgrid(T, gh + (units + T - 1) / T);
+    const dim3 vgrid(T, (wide ? 1 : gh) + (units + T - 1) / T);
+    if (wide) {
+      const int np = ((Hq + Hkv) * dim + NT * 8 - 1) / (NT * 8);
+#define SM_QWC(NP)                                                                                                    \
+  hipLaunchKernelGGL(qkv_wide_cache_vec_kernel<NP>, vgrid, dim3(NT), 0, stream, (const bf16_t*)qkv, stride, bias,     \
+                     positions, cos_sin, Hq, Hkv, dim, vdim, rot_dims, eps, v_first, v_mode, lam, slots,              \
+                     (bf16_t*)cache, bs, (bf16_t*)q_out, qk_w, cvh, tg, T, q_scale)
+      if (np <= 1) SM_QWC(1);
+      else if (np <= 2) SM_QWC(2);
+      else if (np <= 4) SM_QWC(4);
+      else SM_QWC(8);
+#undef SM_QWC
+      return;
+    }
 #define SM_QRC(N)                                                                                                     \
   case N:                                                                                                             \
     hipLaunchKernelGGL(qkv_rope_cache_vec_kernel<N>, vgrid, dim3(NT), 0, stream, (const bf16_t*)qkv, stride, bias,    \
                        positions, cos_sin, Hq, Hkv, dim, vdim, rot_dims, interleaved, unit, eps, v_first, v_mode, lam, \
-                       slots, (bf16_t*)cache, bs, (bf16_t*)q_out, qk_w, norm_first, v_from_k, cvh, gh, tg, T, wide,   \
+                       slots, (bf16_t*)cache, bs, (bf16_t*)q_out, qk_w, norm_first, v_from_k, cvh, gh, tg, T,         \
                        q_scale);                                                                                      \
     break
     switch (taps) {

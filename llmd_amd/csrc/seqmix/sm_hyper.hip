@@ -200,11 +200,11 @@ __global__ __launch_bounds__(NT) void hyper_update_norm_vec_kernel(float* __rest
 }
 
 // KIND 0: gelu_tanh(g) v; 1: silu(g) v; 2: the clamped units.
-template <int KIND>
+template <typename T, int KIND>
 __device__ __forceinline__ float gate1(float g, float v, float limit) {
   if (KIND == 0) return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * v;
   if (KIND == 1) return g / (1.f + expf(-g)) * v;
-  return clamped_unit(g, v, limit);
+  return clamped_unit<T>(g, v, limit);
 }
 
 template <typename T, int KIND>
@@ -214,7 +214,7 @@ __global__ __launch_bounds__(NT) void gated_act_kernel(const T* __restrict__ gu,
   if (i >= n) return;
   const int64_t t = i / F;
   const int j = (int)(i - t * F);
-  st(out + i, gate1<KIND>(ld(gu + t * stride + j), ld(gu + t * stride + F + j), limit));
+  st(out + i, gate1<T, KIND>(ld(gu + t * stride + j), ld(gu + t * stride + F + j), limit));
 }
 
 // bf16, F % 8 == 0, 16-byte aligned rows: eight columns per thread from 16-byte loads.
@@ -232,7 +232,7 @@ __global__ __launch_bounds__(NT) void gated_act_vec_kernel(const bf16_t* __restr
   ld4(gu + t * stride + F + j, *reinterpret_cast<float(*)[4]>(&v[0]));
   ld4(gu + t * stride + F + j + 4, *reinterpret_cast<float(*)[4]>(&v[4]));
 #pragma unroll
-  for (int q = 0; q < 8; ++q) o[q] = gate1<KIND>(g[q], v[q], limit);
+  for (int q = 0; q < 8; ++q) o[q] = gate1<bf16_t, KIND>(g[q], v[q], limit);
   st4(out + t * F + j, *reinterpret_cast<float(*)[4]>(&o[0]));
   st4(out + t * F + j + 4, *reinterpret_cast<float(*)[4]>(&o[4]));
 }

@@ -322,9 +322,9 @@ __device__ __forceinline__ float gelu_tanh_(float v) {
   return 0.5f * v * (1.f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
 }
 constexpr bool gated_act_code(int act) { return act == 2 || act == 3 || act == 5; }
-template <int ACT>
+template <typename T, int ACT>
 __device__ __forceinline__ float gated_(float g, float u, float limit) {
-  if (ACT == 5) return clamped_unit(g, u, limit);
+  if (ACT == 5) return clamped_unit<T>(g, u, limit);
   return (ACT == 2 ? gelu_tanh_(g) : g / (1.f + expf(-g))) * u;
 }
 
@@ -389,7 +389,7 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const T* __restrict__ A, 
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         const int n = n0 + tx * 2 + j;
-        if (n < N) st(Cout + (int64_t)(slot0 + r) * N + n, gated_<ACT>(sw[r] * acc[i][j], sw[r] * acc[i][j + 2], limit));
+        if (n < N) st(Cout + (int64_t)(slot0 + r) * N + n, gated_<T, ACT>(sw[r] * acc[i][j], sw[r] * acc[i][j + 2], limit));
       }
       continue;
     }
@@ -529,7 +529,7 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_kernel(const bf16_t* __rest
           const int n = n0 + wn * 8 * NJ + j * 16 + r16;
           if (n < N)
             st(Cout + (int64_t)(slot0 + row) * N + n,
-               gated_<ACT>(sw[row] * acc[i][j][r], sw[row] * acc[i][j + NJ / 2][r], limit));
+               gated_<bf16_t, ACT>(sw[row] * acc[i][j][r], sw[row] * acc[i][j + NJ / 2][r], limit));
         }
         continue;
       }

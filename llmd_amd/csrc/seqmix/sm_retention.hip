@@ -29,7 +29,7 @@ namespace {
 constexpr int NT = 256;
 constexpr int C = 64;         // tokens per chunk
 constexpr int DB = 64;        // key dimensions staged at a time
-constexpr int QS = DB + 4;    // LDS row stride of q and k
+constexpr int QS = DB + 4;    // LDS row stride of the keys
 constexpr int MAXCOLS = 256;  // value columns of a workgroup
 
 typedef float f32x4_t __attribute__((ext_vector_type(4)));
@@ -62,25 +62,29 @@ __device__ __forceinline__ float rot1(const T* row, int e, const float* cs, int 
   return first ? x * c - xp * s : x * c + xp * s;
 }
 
-// Elements e .. e + 3 (vec: e, half and dk multiples of four, rows aligned for it); elements past dk are zero.
-template <typename T>
-__device__ __forceinline__ void rot4(const T* row, int e, int dk, const float* cs, int half, bool vec, float (&v)[4]) {
-  if (!vec) {
+// Elements e .. e + 3, zero past dk. VEC (dk and half multiples of four, rows aligned for it): all loads are
+// unconditional, from clamped places, so that those of several calls are in flight together.
+template <typename T, bool VEC>
+__device__ __forceinline__ void rot4(const T* row, int e, int dk, const float* cs, int half, float (&v)[4]) {
+  if constexpr (!VEC) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) v[i] = e + i < dk ? rot1(row, e + i, cs, half) : 0.f;
-    return;
-  }
-  v[0] = v[1] = v[2] = v[3] = 0.f;
-  if (e >= dk) return;
-  ld4(row + e, v);
-  if (e >= 2 * half) return;
-  const bool first = e < half;
-  float p[4], c[4], s[4];
-  ld4(row + (first ? e + half : e - half), p);
-  ld4(cs + (first ? e : e - half), c);
-  ld4(cs + half + (first ? e : e - half), s);
+  } else {
+    const int ec = min(e, dk - 4);
+    ld4(row + ec, v);
+    if (half > 0) {
+      const bool first = ec < half, in = ec < 2 * half;
+      const int f = in ? (first ? ec : ec - half) : 0;
+      float p[4], c[4], s[4];
+      ld4(row + (in ? (first ? ec + half : ec - half) : ec), p);
+      ld4(cs + f, c);
+      ld4(cs + half + f, s);
 #pragma unroll
-  for (int i = 0; i < 4; ++i) v[i] = first ? v[i] * c[i] - p[i] * s[i] : v[i] * c[i] + p[i] * s[i];
+      for (int i = 0; i < 4; ++i) v[i] = in ? (first ? v[i] * c[i] - p[i] * s[i] : v[i] * c[i] + p[i] * s[i]) : v[i];
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = e < dk ? v[i] : 0.f;
+  }
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -97,42 +101,49 @@ __global__ __launch_bounds__(NT) void retention_step_kernel(const T* __restrict_
   __shared__ float red[NT / 64];
   const int h = blockIdx.x, s = blockIdx.y;
   const int64_t t = seq_start[s];
+  const bool init = seq_init[s] != 0;
+  float* sp = state + ((int64_t)seq_slot[s] * H + h) * dk * dv;
   float *sq = lds, *sk = lds + dk, *so = lds + 2 * dk;  // so [RG, dv]
   const T* row = p + t * stride;
+  const int rg = threadIdx.x / ncg, cg = threadIdx.x - rg * ncg;
+  constexpr int U = 8;  // rows of the state in flight
+  float S[U][VEC];
+  auto load = [&](int r0, int col) {
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int r = r0 + u * RG;
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) S[u][i] = 0.f;
+      if (init && r < dk) {
+        if constexpr (VEC == 4) ld4(sp + (int64_t)r * dv + col, S[u]);
+        else S[u][0] = sp[(int64_t)r * dv + col];
+      }
+    }
+  };
+  if (rg < RG) load(rg, cg * VEC);  // the first piece is on its way while the keys and queries are rotated
   const int half = rot.dims >> 1;
   const float* cs = rot.dims ? rot.cos_sin + rot.positions[t] * rot.dims : nullptr;
   const float kscale = 1.f / sqrtf((float)dk);
-  for (int e = threadIdx.x; e < dk; e += NT) {
-    sq[e] = rot1(row + h * dk, e, cs, half);
-    sk[e] = rot1(row + (H + h) * dk, e, cs, half) * kscale;
+  const float decay = powers[h * pw_stride + 1];
+  for (int e = threadIdx.x; e < 2 * dk; e += NT) {
+    const bool is_q = e < dk;
+    const int d = is_q ? e : e - dk;
+    const float x = rot1(row + (is_q ? h : H + h) * dk, d, cs, half);
+    lds[e] = is_q ? x : x * kscale;
   }
   __syncthreads();
-  const bool init = seq_init[s] != 0;
-  const float decay = powers[h * pw_stride + 1];
-  float* sp = state + ((int64_t)seq_slot[s] * H + h) * dk * dv;
   const T* vrow = row + 2 * H * dk + h * dv;
-  const int rg = threadIdx.x / ncg, cg = threadIdx.x - rg * ncg;
   if (rg < RG) {
     for (int col = cg * VEC; col < dv; col += ncg * VEC) {
+      if (col != cg * VEC) load(rg, col);
       float v[VEC], o[VEC];
 #pragma unroll
       for (int i = 0; i < VEC; ++i) {
         v[i] = ld(vrow + col + i);
         o[i] = 0.f;
       }
-      constexpr int U = 8;  // rows in flight
       for (int r0 = rg; r0 < dk; r0 += RG * U) {
-        float S[U][VEC];
-#pragma unroll
-        for (int u = 0; u < U; ++u) {
-          const int r = r0 + u * RG;
-#pragma unroll
-          for (int i = 0; i < VEC; ++i) S[u][i] = 0.f;
-          if (init && r < dk) {
-            if constexpr (VEC == 4) ld4(sp + (int64_t)r * dv + col, S[u]);
-            else S[u][0] = sp[(int64_t)r * dv + col];
-          }
-        }
+        if (r0 != rg) load(r0, col);
 #pragma unroll
         for (int u = 0; u < U; ++u) {
           const int r = r0 + u * RG;
@@ -154,6 +165,8 @@ __global__ __launch_bounds__(NT) void retention_step_kernel(const T* __restrict_
     }
   }
   __syncthreads();
+  const T* grow = row + 2 * H * dk + H * dv + h * dv;
+  const float g0 = gate && (int)threadIdx.x < dv ? ld(grow + threadIdx.x) : 0.f;
   float ss = 0.f;
   for (int e = threadIdx.x; e < dv; e += NT) {  // a thread reads back only what it sums here
     float a = 0.f;
@@ -164,40 +177,42 @@ __global__ __launch_bounds__(NT) void retention_step_kernel(const T* __restrict_
   const float inv = 1.f / sqrtf(block_sum<NT>(ss, red) / (float)dv + eps);
   for (int e = threadIdx.x; e < dv; e += NT) {
     float o = so[e] * inv;
-    if (gate) o *= Fn<T>::silu(ld(row + 2 * H * dk + H * dv + h * dv + e));
+    if (gate) o *= Fn<T>::silu(e < NT ? g0 : ld(grow + e));
     st(out + (t * H + h) * dv + e, o);
   }
 }
 
 // ---------------------------------------------------------------------------------------------
-// Stage CB value columns [col0, col0 + CB) of tokens t0 .. t0 + n - 1 (rows past n and columns past dv are zero).
-template <typename T, int CB>
+// Stage CB value columns [col0, col0 + CB) of ROWS tokens t0 .. (rows past n and columns past dv are zero).
+template <typename T, int CB, int ROWS, bool VEC>
 __device__ __forceinline__ void stage_v(const T* __restrict__ p, int64_t stride, int64_t t0, int n, int voff, int col0,
-                                        int dv, bool vec, float* sV) {
+                                        int dv, float* sV) {
   constexpr int BS = CB + 4;
-  for (int e = threadIdx.x; e < C * (CB / 4); e += NT) {
-    const int j = e / (CB / 4), c = (e - j * (CB / 4)) * 4;
-    float v[4] = {0.f, 0.f, 0.f, 0.f};
-    if (j < n) {
-      const T* src = p + (t0 + j) * stride + voff + col0 + c;
-      if (vec) {
-        if (col0 + c < dv) ld4(src, v);
-      } else {
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
-          if (col0 + c + i < dv) v[i] = ld(src + i);
-      }
+  for (int e0 = 0; e0 < ROWS * (CB / 4); e0 += NT) {
+    const int e = e0 + threadIdx.x;
+    const int j = e / (CB / 4), c = (e - j * (CB / 4)) * 4;
+    const T* src = p + (t0 + min(j, n - 1)) * stride + voff;
+    float v[4] = {0.f, 0.f, 0.f, 0.f};
+    if constexpr (VEC) {
+      ld4(src + min(col0 + c, dv - 4), v);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = j < n && col0 + c < dv ? v[i] : 0.f;
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (j < n && col0 + c + i < dv) v[i] = ld(src + col0 + c + i);
     }
     *reinterpret_cast<float4*>(&sV[j * BS + c]) = make_float4(v[0], v[1], v[2], v[3]);
   }
 }
 
 // L = sum_j decay^(n-1-j) k_j v_j^T of chunk c0 + blockIdx.x, head blockIdx.y; blockIdx.z: block of DB key rows x CB columns.
-template <typename T, int NCB>
+template <typename T, int NCB, bool VEC>
 __global__ __launch_bounds__(NT) void retention_chunk_kernel(const T* __restrict__ p, int64_t stride, int H, int dk,
                                                              int dv, Rot rot, const float* __restrict__ powers,
                                                              int pw_stride, const int* __restrict__ c_start, int c0,
-                                                             float* __restrict__ c_state, int vec) {
+                                                             float* __restrict__ c_state) {
   constexpr int CB = 16 * NCB, BS = CB + 4;
   extern __shared__ __attribute__((aligned(16))) float lds[];
   float *sK = lds, *sV = lds + C * QS;
@@ -209,19 +224,19 @@ __global__ __launch_bounds__(NT) void retention_chunk_kernel(const T* __restrict
   const int half = rot.dims >> 1;
   const float kscale = 1.f / sqrtf((float)dk);
   const float* pw = powers + (int64_t)h * pw_stride;
-  for (int e = threadIdx.x; e < C * (DB / 4); e += NT) {
-    const int j = e / (DB / 4), d = (e - j * (DB / 4)) * 4;
-    float v[4] = {0.f, 0.f, 0.f, 0.f};
-    if (j < n) {
-      const float* cs = rot.dims ? rot.cos_sin + rot.positions[t0 + j] * rot.dims : nullptr;
-      rot4(p + (t0 + j) * stride + (H + h) * dk, d0 + d, dk, cs, half, vec != 0, v);
-      const float w = kscale * pw[n - 1 - j];
+  const int64_t pos0 = rot.positions[t0];  // a chunk's positions follow each other
 #pragma unroll
-      for (int i = 0; i < 4; ++i) v[i] *= w;
-    }
+  for (int e0 = 0; e0 < C * (DB / 4); e0 += NT) {
+    const int e = e0 + threadIdx.x;
+    const int j = e / (DB / 4), d = (e - j * (DB / 4)) * 4, jc = min(j, n - 1);
+    float v[4];
+    rot4<T, VEC>(p + (t0 + jc) * stride + (H + h) * dk, d0 + d, dk, rot.cos_sin + (pos0 + jc) * rot.dims, half, v);
+    const float w = j < n ? kscale * pw[n - 1 - jc] : 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = j < n ? v[i] * w : 0.f;
     *reinterpret_cast<float4*>(&sK[j * QS + d]) = make_float4(v[0], v[1], v[2], v[3]);
   }
-  stage_v<T, CB>(p, stride, t0, n, 2 * H * dk + h * dv, col0, dv, vec != 0, sV);
+  stage_v<T, CB, C, VEC>(p, stride, t0, n, 2 * H * dk + h * dv, col0, dv, sV);
   __syncthreads();
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int r16 = lane & 15, kq = lane >> 4;
@@ -274,23 +289,23 @@ __global__ __launch_bounds__(NT) void retention_link_kernel(float* __restrict__ 
     if constexpr (VEC == 4) ld4(sp, S);
     else S[0] = sp[0];
   }
-  constexpr int U = 8;  // chunks in flight
+  constexpr int U = 16;  // chunks in flight
+  const float d_full = pw[C], d_last = pw[c_start[hi] - c_start[hi - 1]];  // all chunks but a run's last are whole
   for (int cb = lo; cb < hi; cb += U) {
     float L[U][VEC];
 #pragma unroll
-    for (int u = 0; u < U; ++u)
-      if (cb + u < hi) {
-        const float* src = c_state + (int64_t)(cb + u - c0) * total + e;
-        if constexpr (VEC == 4) ld4(src, L[u]);
-        else L[u][0] = src[0];
-      }
+    for (int u = 0; u < U; ++u) {
+      const float* src = c_state + (int64_t)(min(cb + u, hi - 1) - c0) * total + e;
+      if constexpr (VEC == 4) ld4(src, L[u]);
+      else L[u][0] = src[0];
+    }
 #pragma unroll
     for (int u = 0; u < U; ++u)
       if (cb + u < hi) {
         float* dst = c_state + (int64_t)(cb + u - c0) * total + e;
         if constexpr (VEC == 4) *reinterpret_cast<float4*>(dst) = make_float4(S[0], S[1], S[2], S[3]);
         else dst[0] = S[0];
-        const float d = pw[c_start[cb + u + 1] - c_start[cb + u]];
+        const float d = cb + u == hi - 1 ? d_last : d_full;
 #pragma unroll
         for (int i = 0; i < VEC; ++i) S[i] = d * S[i] + L[u][i];
       }
@@ -300,16 +315,21 @@ __global__ __launch_bounds__(NT) void retention_link_kernel(float* __restrict__ 
 }
 
 // The read-outs of chunk c0 + blockIdx.x, head blockIdx.y, columns CB blockIdx.z ..; c_state holds the chunks' start states.
-template <typename T, int NCB>
-__global__ __launch_bounds__(NT) void retention_out_kernel(const T* __restrict__ p, int64_t stride, int H, int dk,
+// A wave's 16 rotated queries go from global memory to its registers; keys (OB dimensions at a time), the state's
+// rows (OB at a time) and the values (OB tokens at a time) pass through LDS in small pieces, so that several
+// workgroups share a CU and hide each other's loads.
+constexpr int OB = 32, OS = OB + 4;
+
+template <typename T, int NCB, bool VEC>
+__global__ __launch_bounds__(NT, NCB <= 4 ? 4 : NCB <= 8 ? 3 : 2) void retention_out_kernel(const T* __restrict__ p, int64_t stride, int H, int dk,
                                                            int dv, int gate, Rot rot, const float* __restrict__ powers,
                                                            int pw_stride, float eps, const int* __restrict__ c_start,
                                                            int c0, const float* __restrict__ c_state,
-                                                           T* __restrict__ out, float* __restrict__ o_raw, int vec) {
+                                                           T* __restrict__ out, float* __restrict__ o_raw) {
   constexpr int CB = 16 * NCB, BS = CB + 4;
   extern __shared__ __attribute__((aligned(16))) float lds[];
   __shared__ float sP[C + 1];
-  float *sQ = lds, *sK = lds + C * QS, *sB = lds + 2 * C * QS;  // sB [64, CB]: a block of the state, then the values
+  float *sK = lds, *sB = lds + C * OS;  // sK [64 keys, OB]; sB [OB, CB]: a piece of the state, then of the values
   const int c = blockIdx.x, h = blockIdx.y, col0 = blockIdx.z * CB;
   const int64_t t0 = c_start[c0 + c];
   const int n = c_start[c0 + c + 1] - (int)t0;
@@ -319,58 +339,64 @@ __global__ __launch_bounds__(NT) void retention_out_kernel(const T* __restrict__
   const int r16 = lane & 15, kq = lane >> 4;
   if (threadIdx.x <= C) sP[threadIdx.x] = powers[(int64_t)h * pw_stride + threadIdx.x];
   const float* S0 = c_state + ((int64_t)c * H + h) * dk * dv;
+  const int64_t pos0 = rot.positions[t0];  // a chunk's positions follow each other
+  const int qi = wave * 16 + r16, qc = min(qi, n - 1);
+  const T* q_row = p + (t0 + qc) * stride + h * dk;
+  const float* q_cs = rot.cos_sin + (pos0 + qc) * rot.dims;
   f32x4_t o[NCB], w[4];  // o: rows 16 wave + 4 kq + r, column 16 m + r16; w[jb]: key 16 jb + 4 kq + r of query 16 wave + r16
 #pragma unroll
   for (int m = 0; m < NCB; ++m) o[m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int jb = 0; jb < 4; ++jb) w[jb] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  for (int d0 = 0; d0 < dk; d0 += DB) {
-    if (d0 > 0) __syncthreads();  // the previous block is read
-    for (int e = threadIdx.x; e < C * (DB / 4); e += NT) {
-      const int j = e / (DB / 4), d = (e - j * (DB / 4)) * 4;
-      float a[4] = {0.f, 0.f, 0.f, 0.f}, b[4] = {0.f, 0.f, 0.f, 0.f};
-      if (j < n) {
-        const float* cs = rot.dims ? rot.cos_sin + rot.positions[t0 + j] * rot.dims : nullptr;
-        const T* row = p + (t0 + j) * stride;
-        rot4(row + h * dk, d0 + d, dk, cs, half, vec != 0, a);
-        rot4(row + (H + h) * dk, d0 + d, dk, cs, half, vec != 0, b);
-      }
-      *reinterpret_cast<float4*>(&sQ[j * QS + d]) = make_float4(a[0], a[1], a[2], a[3]);
-      *reinterpret_cast<float4*>(&sK[j * QS + d]) = make_float4(b[0] * kscale, b[1] * kscale, b[2] * kscale, b[3] * kscale);
-    }
-    for (int e = threadIdx.x; e < DB * (CB / 4); e += NT) {
-      const int d = e / (CB / 4), cc = (e - d * (CB / 4)) * 4;
-      float v[4] = {0.f, 0.f, 0.f, 0.f};
-      if (d0 + d < dk) {
-        const float* src = S0 + (int64_t)(d0 + d) * dv + col0 + cc;
-        if (vec) {
-          if (col0 + cc < dv) ld4(src, v);
-        } else {
+  for (int d0 = 0; d0 < dk; d0 += OB) {
+    float a[OB / 16][4];  // this lane's query, dimensions d0 + 16 i + 4 kq .. (a row past n repeats the last one)
 #pragma unroll
-          for (int i = 0; i < 4; ++i)
-            if (col0 + cc + i < dv) v[i] = src[i];
-        }
+    for (int i = 0; i < OB / 16; ++i) rot4<T, VEC>(q_row, d0 + 16 * i + 4 * kq, dk, q_cs, half, a[i]);
+    if (d0 > 0) __syncthreads();  // the previous piece is read
+#pragma unroll
+    for (int e0 = 0; e0 < C * (OB / 4); e0 += NT) {
+      const int e = e0 + threadIdx.x;
+      const int j = e / (OB / 4), d = (e - j * (OB / 4)) * 4, jc = min(j, n - 1);
+      float b[4];
+      rot4<T, VEC>(p + (t0 + jc) * stride + (H + h) * dk, d0 + d, dk, rot.cos_sin + (pos0 + jc) * rot.dims, half, b);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) b[i] = j < n ? b[i] * kscale : 0.f;
+      *reinterpret_cast<float4*>(&sK[j * OS + d]) = make_float4(b[0], b[1], b[2], b[3]);
+    }
+#pragma unroll
+    for (int e0 = 0; e0 < OB * (CB / 4); e0 += NT) {
+      const int e = e0 + threadIdx.x;
+      const int d = e / (CB / 4), cc = (e - d * (CB / 4)) * 4;
+      const float* src = S0 + (int64_t)min(d0 + d, dk - 1) * dv;
+      float v[4] = {0.f, 0.f, 0.f, 0.f};
+      if constexpr (VEC) {
+        ld4(src + min(col0 + cc, dv - 4), v);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = d0 + d < dk && col0 + cc < dv ? v[i] : 0.f;
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (d0 + d < dk && col0 + cc + i < dv) v[i] = src[col0 + cc + i];
       }
       *reinterpret_cast<float4*>(&sB[d * BS + cc]) = make_float4(v[0], v[1], v[2], v[3]);
     }
     __syncthreads();
-    const int dn = min(DB, dk - d0);
-    for (int s16 = 0; s16 < dn; s16 += 16) {
-      float a[4];
-      ld4(&sQ[(wave * 16 + r16) * QS + s16 + 4 * kq], a);
+#pragma unroll
+    for (int i = 0; i < OB / 16; ++i) {
+      if (d0 + 16 * i >= dk) break;
 #pragma unroll
       for (int jb = 0; jb < 4; ++jb) {
         if (jb > wave) break;  // keys after every query of this wave
         float b[4];
-        ld4(&sK[(jb * 16 + r16) * QS + s16 + 4 * kq], b);
+        ld4(&sK[(jb * 16 + r16) * OS + 16 * i + 4 * kq], b);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) w[jb] = __builtin_amdgcn_mfma_f32_16x16x4f32(b[e], a[e], w[jb], 0, 0, 0);
+        for (int e = 0; e < 4; ++e) w[jb] = __builtin_amdgcn_mfma_f32_16x16x4f32(b[e], a[i][e], w[jb], 0, 0, 0);
       }
 #pragma unroll
       for (int e = 0; e < 4; ++e)
 #pragma unroll
         for (int m = 0; m < NCB; ++m)
-          o[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], sB[(s16 + 4 * kq + e) * BS + m * 16 + r16], o[m], 0, 0, 0);
+          o[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i][e], sB[(16 * i + 4 * kq + e) * BS + m * 16 + r16], o[m], 0, 0, 0);
     }
   }
   // decay of the state's part by the row, of a weight by the distance
@@ -387,17 +413,22 @@ __global__ __launch_bounds__(NT) void retention_out_kernel(const T* __restrict__
       const int dist = wave * 16 + r16 - (jb * 16 + kq * 4 + r);
       w[jb][r] = dist >= 0 ? w[jb][r] * sP[max(dist, 0)] : 0.f;
     }
-  __syncthreads();  // the last block of the state is read
-  stage_v<T, CB>(p, stride, t0, n, 2 * H * dk + h * dv, col0, dv, vec != 0, sB);
-  __syncthreads();
 #pragma unroll
-  for (int jb = 0; jb < 4; ++jb) {
-    if (jb > wave) break;
+  for (int j0 = 0; j0 < C; j0 += OB) {
+    if (j0 >= n) break;
+    __syncthreads();  // the previous piece is read
+    stage_v<T, CB, OB, VEC>(p, stride, t0 + j0, n - j0, 2 * H * dk + h * dv, col0, dv, sB);
+    __syncthreads();
 #pragma unroll
-    for (int e = 0; e < 4; ++e)
+    for (int i = 0; i < OB / 16; ++i) {
+      const int jb = j0 / 16 + i;
+      if (jb > wave) break;
 #pragma unroll
-      for (int m = 0; m < NCB; ++m)
-        o[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(w[jb][e], sB[(jb * 16 + 4 * kq + e) * BS + m * 16 + r16], o[m], 0, 0, 0);
+      for (int e = 0; e < 4; ++e)
+#pragma unroll
+        for (int m = 0; m < NCB; ++m)
+          o[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(w[jb][e], sB[(16 * i + 4 * kq + e) * BS + m * 16 + r16], o[m], 0, 0, 0);
+    }
   }
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
@@ -419,14 +450,19 @@ __global__ __launch_bounds__(NT) void retention_out_kernel(const T* __restrict__
 #pragma unroll
     for (int x = 8; x > 0; x >>= 1) ss += __shfl_xor(ss, x, 64);
     const float inv = 1.f / sqrtf(ss / (float)dv + eps);
+    float g[NCB];  // the row's gates: loads from clamped places, all in flight together
+    if (gate) {
+      const T* grow = p + (t0 + min(i, n - 1)) * stride + 2 * H * dk + H * dv + h * dv;
+#pragma unroll
+      for (int m = 0; m < NCB; ++m) g[m] = ld(grow + min(m * 16 + r16, dv - 1));
+#pragma unroll
+      for (int m = 0; m < NCB; ++m) o[m][r] *= Fn<T>::silu(g[m]);
+    }
     if (i >= n) continue;
 #pragma unroll
     for (int m = 0; m < NCB; ++m) {
       const int col = m * 16 + r16;
-      if (col >= dv) continue;
-      float v = o[m][r] * inv;
-      if (gate) v *= Fn<T>::silu(ld(p + t * stride + 2 * H * dk + H * dv + h * dv + col));
-      st(out + (t * H + h) * dv + col, v);
+      if (col < dv) st(out + (t * H + h) * dv + col, o[m][r] * inv);
     }
   }
 }
@@ -478,19 +514,23 @@ int launch(const T* p, int64_t stride, int H, int dk, int dv, int gate, const Ro
   auto set = [](const void* k, size_t lds) {
     if (lds > 64 * 1024) (void)hipFuncSetAttribute(k, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
   };
-#define SM_CHUNK(NCB)                                                                                                 \
+#define SM_CHUNK(NCB, VEC)                                                                                            \
   {                                                                                                                   \
     const size_t lds = (size_t)(C * QS + C * (16 * NCB + 4)) * sizeof(float);                                         \
     const dim3 grid(n, H, ((dk + DB - 1) / DB) * ((dv + 16 * NCB - 1) / (16 * NCB)));                                 \
-    set((const void*)retention_chunk_kernel<T, NCB>, lds);                                                            \
-    hipLaunchKernelGGL((retention_chunk_kernel<T, NCB>), grid, dim3(NT), lds, stream, p, stride, H, dk, dv, rot, powers, \
-                       pw_stride, c_start, nd, c_state, vec ? 1 : 0);                                                 \
+    set((const void*)retention_chunk_kernel<T, NCB, VEC>, lds);                                                       \
+    hipLaunchKernelGGL((retention_chunk_kernel<T, NCB, VEC>), grid, dim3(NT), lds, stream, p, stride, H, dk, dv, rot, \
+                       powers, pw_stride, c_start, nd, c_state);                                                      \
   }
-  if (dv <= 64) SM_CHUNK(4)
-  else SM_CHUNK(8)
+  if (dv <= 64 && vec) SM_CHUNK(4, true)
+  else if (dv <= 64) SM_CHUNK(4, false)
+  else if (vec) SM_CHUNK(8, true)
+  else SM_CHUNK(8, false)
 #undef SM_CHUNK
   const int64_t per_head = (int64_t)dk * dv;
-  if (per_head % 4 == 0 && ((uintptr_t)state & 15) == 0 && ((uintptr_t)c_state & 15) == 0)
+  // 16-byte pieces when that still leaves enough threads to fill the chip
+  if (per_head % 4 == 0 && per_head * H * (nseq - nd) >= (int64_t)4 * 65536 && ((uintptr_t)state & 15) == 0 &&
+      ((uintptr_t)c_state & 15) == 0)
     hipLaunchKernelGGL((retention_link_kernel<4>), dim3((unsigned)((per_head * H / 4 + NT - 1) / NT), nseq - nd), dim3(NT),
                        0, stream, c_state, c_start, s_chunk0, nd, nd, H, per_head, powers, pw_stride, state, seq_slot,
                        seq_init);
@@ -498,17 +538,21 @@ int launch(const T* p, int64_t stride, int H, int dk, int dv, int gate, const Ro
     hipLaunchKernelGGL((retention_link_kernel<1>), dim3((unsigned)((per_head * H + NT - 1) / NT), nseq - nd), dim3(NT), 0,
                        stream, c_state, c_start, s_chunk0, nd, nd, H, per_head, powers, pw_stride, state, seq_slot,
                        seq_init);
-#define SM_OUT(NCB)                                                                                                   \
+#define SM_OUT(NCB, VEC)                                                                                              \
   {                                                                                                                   \
-    const size_t lds = (size_t)(2 * C * QS + C * (16 * NCB + 4)) * sizeof(float);                                     \
+    const size_t lds = (size_t)(C * OS + OB * (16 * NCB + 4)) * sizeof(float);                                        \
     const dim3 grid(n, H, (dv + 16 * NCB - 1) / (16 * NCB));                                                          \
-    set((const void*)retention_out_kernel<T, NCB>, lds);                                                              \
-    hipLaunchKernelGGL((retention_out_kernel<T, NCB>), grid, dim3(NT), lds, stream, p, stride, H, dk, dv, gate, rot,   \
-                       powers, pw_stride, eps, c_start, nd, c_state, out, o_raw, vec ? 1 : 0);                        \
+    set((const void*)retention_out_kernel<T, NCB, VEC>, lds);                                                         \
+    hipLaunchKernelGGL((retention_out_kernel<T, NCB, VEC>), grid, dim3(NT), lds, stream, p, stride, H, dk, dv, gate,  \
+                       rot, powers, pw_stride, eps, c_start, nd, c_state, out, o_raw);                                \
   }
-  if (dv <= 64) SM_OUT(4)
-  else if (dv <= 128) SM_OUT(8)
-  else SM_OUT(16)
+#define SM_OUT2(VEC)                  \
+  if (dv <= 64) SM_OUT(4, VEC)        \
+  else if (dv <= 128) SM_OUT(8, VEC)  \
+  else SM_OUT(16, VEC)
+  if (vec) { SM_OUT2(true) }
+  else { SM_OUT2(false) }
+#undef SM_OUT2
 #undef SM_OUT
   if (o_raw != nullptr) {
     const int rows = T_rows - nd;  // the longer runs' tokens follow the nd single ones

@@ -53,6 +53,19 @@ their own, each result behind an element-wise gate of width x width):
   kokatar-hybrid : width 2048, window attention 32 / 4 heads and latent attention in turn, dense and experts
                    in turn
 
+Five Koduzen stacks (two hyper-connected streams with RMS norms, clamped gated units):
+
+  koduzen-window    : width 4096, windowed attention 32 heads / 8 kv heads x 128 (window 1024, norms over whole
+                      projections, ramp-scaled rotation), dense ff 14336 - beside ``negunex-dense`` (same heads,
+                      ff and streams), ``kakalorn-window`` and Llama-3-8B layers
+  koduzen-bias      : the same sizes without rotation (distance bias, query temperature, sinks), every second layer
+                      over the keys and values of the one before it
+  koduzen-retention : width 2048, retention 32 heads x 64 (key) x 64 (value); dense ff 5632 - beside
+                      ``kakalorn-hgrn2`` (same heads and sizes)
+  koduzen-moe       : width 2048, windowed attention 32 heads / 4 kv heads x 128; 128 experts + 4 identity in 4
+                      groups, 2 kept, 8 chosen, ff 768, shared expert 1536 - beside ``negunex-moe``
+  koduzen-hybrid    : width 2048, retention 16 heads x 128 x 256, the two kinds of attention and shared keys in turn
+
 Prefill: one prompt of ``--tokens`` tokens in one step. Decode: ``--batch`` sequences with that
 context, one token each. One JSON line with tokens/s and ms per layer for every entry.
 """
@@ -179,6 +192,39 @@ def _kokatar(kind: str):
                                                 for i in range(n)]})
 
 
+def _koduzen(kind: str):
+    from llmd_amd.engine.config import koduzen_config
+
+    wide = kind in ("window", "bias")
+    heads = {"heads": 32, "kv_heads": 8 if wide else 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+             "mask": {"size": 1024}}
+    rot = {"dims": 128, "base": 500000.0}
+    win = {"type": "attention",
+           "mixer": dict(heads, rot=dict(rot, scaling={"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}))}
+    bias = {"type": "attention_2", "mixer": dict(heads, q_temp={"coef": 0.1, "every": 8192})}
+
+    def ret(h, dim, vdim):
+        return {"type": "retention",
+                "mixer": {"heads": h, "dim": dim, "vdim": vdim, "rot": {"dims": dim, "base": 10000.0},
+                          "decay": [1.0 - 2.0 ** (-5.0 - 3.0 * i / (h - 1)) for i in range(h)]}}
+
+    dense = {"kind": "dense", "ff": 14336 if wide else 5632, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": 768, "limit": 7.0}, "shared": {"ff": 1536, "limit": 7.0},
+           "router": {"experts": 128, "identity": 4, "top": 8, "groups": {"count": 4, "keep": 2}, "scale": 1.0}}
+
+    def make(n):
+        todo = {"window": [(win, dense)], "bias": [(bias, dense), (bias, dense)], "retention": [(ret(32, 64, 64), dense)],
+                "moe": [(win, moe)], "hybrid": [(ret(16, 128, 256), dense), (win, moe), (bias, moe), (bias, dense)]}[kind]
+        layers = [dict(json.loads(json.dumps(todo[i % len(todo)][0])), mlp=todo[i % len(todo)][1]) for i in range(n)]
+        for i in range(1, n):  # the second of two position-free layers reads the first one's keys and values
+            if layers[i]["type"] == layers[i - 1]["type"] == "attention_2" and "kv_from" not in layers[i - 1]["mixer"]:
+                layers[i]["mixer"]["kv_from"] = i - 1
+        return koduzen_config({"architecture": "Koduzen", "name": "koduzen-" + kind, "width": 4096 if wide else WIDTH,
+                               "vocab": 32000, "norm": {"eps": 1e-6}, "streams": 2, "layers": layers})
+
+    return make
+
+
 def _runner(mc, tokens: int, batch: int, device: str):
     from llmd_amd.engine.config import EngineConfig
     from llmd_amd.engine.model_runner import ModelRunner
@@ -250,6 +296,7 @@ def run(tokens: int = 2048, batch: int = 32, n_layers: int = 4, reps: int = 5, d
             ("kakalorn-hgrn2", _kakalorn("hgrn2")(n_layers), n_layers),
             ("kakalorn-hybrid", _kakalorn("hybrid")(n_layers), n_layers)]
     todo += [("kokatar-" + k, _kokatar(k)(n_layers), n_layers) for k in ("window", "latent", "moe", "hybrid")]
+    todo += [("koduzen-" + k, _koduzen(k)(n_layers), n_layers) for k in ("window", "bias", "retention", "moe", "hybrid")]
     for name, mc, L in todo:
         if only and not any(name.startswith(o) for o in only.split(",")):
             continue

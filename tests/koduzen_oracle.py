@@ -90,18 +90,21 @@ def softmax_rows(q, k, v, scale, size=None, sink=None, slope=0.0):
     return out
 
 
-def attention(h, W, pre, m, eps):
-    """Grouped attention: norms over whole projections, partial rotation, a window."""
+def attention(h, W, pre, m, eps, kv=None):
+    """Grouped attention: norms over whole projections, partial rotation, a window; ``kv`` the (rotated) keys and the
+    values of another layer. Returns (result, (k, v))."""
     T = h.shape[0]
     H, G, d, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
     q = rms_norm(linear(h, W, pre + "q"), eps, W[pre + "q.norm"]).view(T, H, d)
-    k = rms_norm(linear(h, W, pre + "k"), eps, W[pre + "k.norm"]).view(T, G, d)
-    v = linear(h, W, pre + "v").view(T, G, dv)
     rot = m["rot"]
-    q, k = (rotate(t, rot["dims"], rot["base"], rot.get("scaling")) for t in (q, k))
+    q = rotate(q, rot["dims"], rot["base"], rot.get("scaling"))
+    if kv is None:
+        k = rms_norm(linear(h, W, pre + "k"), eps, W[pre + "k.norm"]).view(T, G, d)
+        kv = rotate(k, rot["dims"], rot["base"], rot.get("scaling")), linear(h, W, pre + "v").view(T, G, dv)
+    k, v = kv
     size = m["mask"]["size"]
     o = [softmax_rows(q[:, n], k[:, n // (H // G)], v[:, n // (H // G)], m["scale"], size) for n in range(H)]
-    return linear(torch.cat(o, -1), W, pre + "o")
+    return linear(torch.cat(o, -1), W, pre + "o"), kv
 
 
 def attention_2(h, W, pre, m, kv=None):
@@ -198,12 +201,14 @@ def forward(cfg, W, tokens, layers_out=None):
             h = rms_norm(u, eps, W[pre + "norm1"])
             if spec["type"] == "retention":
                 return retention(h, W, pre + "mix.", m, eps)
+            kv = kvs[m["kv_from"]] if "kv_from" in m else None
             if spec["type"] == "attention":
-                return attention(h, W, pre + "mix.", m, eps)
-            if spec["type"] == "attention_2":
-                y, kvs[i] = attention_2(h, W, pre + "mix.", m, kvs[m["kv_from"]] if "kv_from" in m else None)
-                return y
-            raise ValueError(spec["type"])
+                y, kvs[i] = attention(h, W, pre + "mix.", m, eps, kv)
+            elif spec["type"] == "attention_2":
+                y, kvs[i] = attention_2(h, W, pre + "mix.", m, kv)
+            else:
+                raise ValueError(spec["type"])
+            return y
 
         def ff(u):
             h = rms_norm(u, eps, W[pre + "norm2"])
@@ -256,7 +261,8 @@ def random_weights(cfg, seed=0, dtype=torch.float32):
                 mat(mp + "v", m["kv_heads"] * dv, d)
             if spec["type"] == "attention":
                 vec(mp + "q.norm", H * dim)
-                vec(mp + "k.norm", m["kv_heads"] * dim)
+                if "kv_from" not in m:
+                    vec(mp + "k.norm", m["kv_heads"] * dim)
             else:
                 vec(mp + "sink", H, mean=0.0, std=1.0)
         mat(mp + "o", d, H * dv)
