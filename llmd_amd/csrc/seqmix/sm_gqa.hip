@@ -871,7 +871,7 @@ __global__ __launch_bounds__(NT, NKS <= 4 && RB == 1 ? 3 : 1) void grouped_atten
     }
     const bf16_t* const tK = sK + cur * MKT * KS;
     const bf16_t* const tV = sVt + cur * VP * VS;
-    const bool plain = slopes == nullptr && k0 >= full_lo && k0 + MKT <= full_hi;
+    const bool plain = k0 >= full_lo && k0 + MKT <= full_hi;  // every key visible to every row: no masks
     // scores of this lane's rows against keys k0 + 16 kb + 4 kq + r
     float sc[RB][2][4];
 #pragma unroll
@@ -900,6 +900,13 @@ __global__ __launch_bounds__(NT, NKS <= 4 && RB == 1 ? 3 : 1) void grouped_atten
           float& v = sc[rb][i >> 2][i & 3];
           v = in ? v - myslope[rb] * (float)(mylen[rb] - 1 - key) : -INFINITY;
         }
+    } else if (slopes != nullptr) {
+#pragma unroll
+      for (int rb = 0; rb < RB; ++rb) {
+        const float dist = (float)(mylen[rb] - 1 - k0 - kq * 4);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) sc[rb][i >> 2][i & 3] -= myslope[rb] * (dist - (float)((i >> 2) * 16 + (i & 3)));
+      }
     }
     // The weights never pass through LDS. After S^T = K Q^T this lane holds, for its query row r16,
     // the keys 4 kq .. 4 kq + 3 of both 16-key halves of the tile - eight keys, which is exactly one
@@ -1103,7 +1110,7 @@ __global__ __launch_bounds__(NT, NKS <= 2 ? 3 : NKS <= 4 ? 2 : 1) void grouped_d
   };
   const int full_lo = max(lo, wlo);  // tiles from here to the sequence's end need no mask
   auto step = [&](int b, int k0) {
-    const bool plain = slopes == nullptr && k0 >= full_lo && k0 + MKT <= len;
+    const bool plain = k0 >= full_lo && k0 + MKT <= len;
     float sc[8];
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb) {
@@ -1121,6 +1128,10 @@ __global__ __launch_bounds__(NT, NKS <= 2 ? 3 : NKS <= 4 ? 2 : 1) void grouped_d
         const bool in = (key < len) & (key >= lo) & ((key >= wlo) | (key < keep));
         sc[i] = in ? sc[i] - slope * (float)(len - 1 - key) : -INFINITY;
       }
+    } else if (slopes != nullptr) {
+      const float dist = (float)(len - 1 - k0 - 8 * kq);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) sc[i] -= slope * (dist - (float)i);
     }
     float mx = sc[0];
 #pragma unroll
